@@ -23,12 +23,6 @@ torch::Tensor sample_topp(torch::Tensor logits, double temperature, double top_p
                           long seed, long step);
 std::vector<torch::Tensor> sample_topp_dev(torch::Tensor logits, double temperature,
                                            double top_p, long seed, torch::Tensor step);
-// kvcache.hip
-void kv_append(torch::Tensor k, torch::Tensor v, torch::Tensor slots,
-               torch::Tensor k_cache, torch::Tensor v_cache);
-torch::Tensor paged_attn_decode(torch::Tensor q, torch::Tensor k_cache,
-                                torch::Tensor v_cache, torch::Tensor block_tables,
-                                torch::Tensor seq_lens, double scale);
 // masked.hip
 std::vector<torch::Tensor> masked_moments(torch::Tensor v, torch::Tensor mask);
 torch::Tensor whiten_apply(torch::Tensor v, double mean, double invstd, double shift);
@@ -60,8 +54,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("adamw_step", &adamw_step);
   m.def("sample_topp", &sample_topp);
   m.def("sample_topp_dev", &sample_topp_dev);
-  m.def("kv_append", &kv_append);
-  m.def("paged_attn_decode", &paged_attn_decode);
   m.def("masked_moments", &masked_moments);
   m.def("whiten_apply", &whiten_apply);
   m.def("lora_gemm", &lora_gemm, py::arg("x"), py::arg("w"),

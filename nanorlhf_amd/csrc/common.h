@@ -30,6 +30,78 @@ DEVINL short f2bf(float f) {
   return (short)(c.u >> 16);
 }
 
+// ---- element access shared by kernels templated on bf16 (short) / float ----
+DEVINL float ldf(const short* p) { return bf2f(*p); }
+DEVINL float ldf(const float* p) { return *p; }
+DEVINL void stf(short* p, float v) { *p = f2bf(v); }
+DEVINL void stf(float* p, float v) { *p = v; }
+
+// VEC consecutive elements as float; VEC > 1 needs VEC-element alignment
+template <int VEC>
+DEVINL void ldv(const float* p, float* o) {
+  if constexpr (VEC % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4) {
+      f32x4 v = *reinterpret_cast<const f32x4*>(p + i);
+#pragma unroll
+      for (int j = 0; j < 4; j++) o[i + j] = v[j];
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i++) o[i] = p[i];
+  }
+}
+template <int VEC>
+DEVINL void ldv(const short* p, float* o) {
+  if constexpr (VEC == 8) {
+    s16x8 v = *reinterpret_cast<const s16x8*>(p);
+#pragma unroll
+    for (int j = 0; j < 8; j++) o[j] = bf2f(v[j]);
+  } else if constexpr (VEC == 4) {
+    s16x4 v = *reinterpret_cast<const s16x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; j++) o[j] = bf2f(v[j]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i++) o[i] = bf2f(p[i]);
+  }
+}
+template <int VEC>
+DEVINL void stv(float* p, const float* v) {
+  if constexpr (VEC % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4)
+      *reinterpret_cast<f32x4*>(p + i) = f32x4{v[i], v[i + 1], v[i + 2], v[i + 3]};
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i++) p[i] = v[i];
+  }
+}
+template <int VEC>
+DEVINL void stv(short* p, const float* v) {
+  if constexpr (VEC == 8) {
+    s16x8 o;
+#pragma unroll
+    for (int j = 0; j < 8; j++) o[j] = f2bf(v[j]);
+    *reinterpret_cast<s16x8*>(p) = o;
+  } else if constexpr (VEC == 4) {
+    s16x4 o;
+#pragma unroll
+    for (int j = 0; j < 4; j++) o[j] = f2bf(v[j]);
+    *reinterpret_cast<s16x4*>(p) = o;
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i++) p[i] = f2bf(v[i]);
+  }
+}
+
+// ---- activations (32-bit) -------------------------------------------------
+DEVINL float act_sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+DEVINL float act_silu(float x) { return x / (1.f + expf(-x)); }
+DEVINL float act_gelu_tanh(float x) {
+  return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+}
+
 // ---- wave (64-lane) reductions ------------------------------------------
 DEVINL float wave_sum(float v) {
 #pragma unroll

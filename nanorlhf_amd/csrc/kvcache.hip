@@ -159,28 +159,43 @@ void kv_append(torch::Tensor k, torch::Tensor v, torch::Tensor slots,
 }
 
 // ------------------------------------------------------- decode attention
-template <int D, typename CT>
+// Mask and output options of the general form (EXT); the plain form compiles
+// them away.
+struct DecodeExt {
+  int size;          // sliding window: position i sees j with i - j < size ...
+  int keep;          // ... and every j < keep
+  int V;             // value width of the output (<= DV, the cache's)
+  long ldo;          // output row stride
+  const float* uncs; // [B, V] cos | sin: turn the output's pairs (2m, 2m+1) back
+  int gchunks;       // query-head groups of 16 per kv head
+};
+
+template <int D, int DV, typename CT, bool EXT>
 __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D]
                                     const CT* __restrict__ kc,      // [P, 16, Hkv, D]
-                                    const CT* __restrict__ vc,      // [P, Hkv, D, 16]
+                                    const CT* __restrict__ vc,      // [P, Hkv, DV, 16]
                                     const int* __restrict__ bt,     // [B, maxP]
                                     const int* __restrict__ seq_lens,
-                                    short* __restrict__ out,        // [B, Hq, D]
-                                    int Hq, int Hkv, int maxP, int G, float scale) {
+                                    short* __restrict__ out,        // [B, Hq, DV]
+                                    int Hq, int Hkv, int maxP, int Gq, float scale,
+                                    DecodeExt ext) {
   constexpr int NC = D / 32;
   constexpr int PS = 16;
-  const int b = blockIdx.x / Hkv;
-  const int kvh = blockIdx.x % Hkv;
+  const int unit = EXT ? blockIdx.x / ext.gchunks : blockIdx.x;
+  const int gc = EXT ? blockIdx.x % ext.gchunks : 0;
+  const int b = unit / Hkv;
+  const int kvh = unit % Hkv;
+  const int G = EXT ? min(16, Gq - 16 * gc) : Gq;   // heads of this workgroup
   const int L = seq_lens[b];
   const int lane = threadIdx.x & 63;
   const int wid = threadIdx.x >> 6;
   const int hi = lane >> 4, lo = lane & 15;
-  const int h0 = kvh * G;
+  const int h0 = kvh * Gq + 16 * gc;
 
   __shared__ short Pb[4][16 * 32];          // per-wave P [g][tok] (bf16)
   __shared__ unsigned char Pb8[4][16 * 32]; // per-wave P (fp8 path)
   __shared__ float Lm[4][16], Ls[4][16];    // per-wave (m, s) per row
-  __shared__ float Lacc[4][16][D];          // per-wave O accumulators
+  __shared__ float Lacc[4][16][DV];         // per-wave O accumulators
 
   // Q fragment: lane holds Q[g = lo][32c + 8hi + j]; zero for g >= G.
   // On the fp8 cache path Q is quantized to e4m3 once here and the QK^T
@@ -209,15 +224,20 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
   }
 
   float m[4], s_[4];
-  f32x4 acc_o[D / 16];
+  f32x4 acc_o[DV / 16];
 #pragma unroll
   for (int r = 0; r < 4; r++) { m[r] = -INFINITY; s_[r] = 0.f; }
 #pragma unroll
-  for (int t = 0; t < D / 16; t++) acc_o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int t = 0; t < DV / 16; t++) acc_o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  const int ntiles = (L + 31) / 32;
+  // tiles with a visible key: those of the kept first tokens, then the window's
+  const int win_lo = EXT ? max(0, L - ext.size) : 0;
+  const int win_tile = win_lo / 32;
+  const int kept_tiles = EXT ? min((ext.keep + 31) / 32, win_tile) : 0;
+  const int ntiles = kept_tiles + (L + 31) / 32 - win_tile;
   const int* btb = bt + (long)b * maxP;
-  for (int tile = wid; tile < ntiles; tile += 4) {
+  for (int it = wid; it < ntiles; it += 4) {
+    const int tile = it < kept_tiles ? it : it - kept_tiles + win_tile;
     const int t0 = tile * 32;
     // ---- scores: S[g][tok] over two 16-token subtiles ------------------
     f32x4 sc[2];
@@ -258,7 +278,8 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
       const int ki = t0 + 16 * n + lo;
 #pragma unroll
       for (int r = 0; r < 4; r++)
-        pm[n][r] = (ki < L) ? sc[n][r] * scale : -INFINITY;
+        pm[n][r] = (ki < L && (!EXT || ki >= win_lo || ki < ext.keep))
+                       ? sc[n][r] * scale : -INFINITY;
     }
     float rowmax[4], fac[4];
 #pragma unroll
@@ -291,7 +312,7 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
       s_[r] = s_[r] * fac[r] + x;
     }
 #pragma unroll
-    for (int t = 0; t < D / 16; t++) {
+    for (int t = 0; t < DV / 16; t++) {
 #pragma unroll
       for (int r = 0; r < 4; r++) acc_o[t][r] *= fac[r];
     }
@@ -308,8 +329,8 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
     const int pv_page = btb[min(2 * tile + (hi >> 1), maxP - 1)];
     const int tokoff = 8 * (hi & 1);
 #pragma unroll
-    for (int t = 0; t < D / 16; t++) {
-      const long vaddr = (((long)pv_page * Hkv + kvh) * D + 16 * t + lo) * PS + tokoff;
+    for (int t = 0; t < DV / 16; t++) {
+      const long vaddr = (((long)pv_page * Hkv + kvh) * DV + 16 * t + lo) * PS + tokoff;
       if (FP8) {
         const long vf8 = load_frag8_raw((const unsigned char*)vc, vaddr);
         acc_o[t] = mfma16k_fp8(pf8, vf8, acc_o[t]);
@@ -327,13 +348,13 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
     for (int r = 0; r < 4; r++) {
       if (lo == 0) { Lm[wid][4 * hi + r] = m[r]; Ls[wid][4 * hi + r] = s_[r]; }
 #pragma unroll
-      for (int t = 0; t < D / 16; t++)
+      for (int t = 0; t < DV / 16; t++)
         Lacc[wid][4 * hi + r][16 * t + lo] = acc_o[t][r];
     }
   }
   __syncthreads();
   if (wid == 0) {
-    constexpr int OV = D / 64;
+    constexpr int OV = DV / 64;
     for (int g = 0; g < G; g++) {
       float M = Lm[0][g];
       for (int w = 1; w < 4; w++) M = fmaxf(M, Lm[w][g]);
@@ -349,17 +370,42 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
 #pragma unroll
           for (int j = 0; j < (OV > 0 ? OV : 1); j++)
             o[j] += Lacc[w][g][lane * OV + j] * c;
-        } else if (lane < D) {
+        } else if (lane < DV) {
           o[0] += Lacc[w][g][lane] * c;
         }
       }
       const float invS = S > 0.f ? 1.f / S : 0.f;
-      short* op = out + ((long)b * Hq + h0 + g) * D;
+      if constexpr (EXT) {
+        short* op = out + (long)b * ext.ldo + (long)(h0 + g) * ext.V;
+        const float* cs = ext.uncs ? ext.uncs + (long)b * ext.V : nullptr;
+        constexpr int NO = OV > 0 ? OV : 1;
+#pragma unroll
+        for (int j = 0; j < NO; j++) o[j] *= invS;
+        if (cs) {
+          const int half = ext.V / 2;
+          float tw[NO];
+#pragma unroll
+          for (int j = 0; j < NO; j++) {
+            const int d = lane * NO + j;
+            const float other = NO > 1 ? o[j ^ 1] : __shfl_xor(o[j], 1);
+            const int pr = min(d >> 1, half - 1);
+            const float c = cs[pr], s = cs[half + pr];
+            tw[j] = o[j] * c + ((d & 1) ? -other : other) * s;
+          }
+#pragma unroll
+          for (int j = 0; j < NO; j++) o[j] = tw[j];
+        }
+#pragma unroll
+        for (int j = 0; j < NO; j++)
+          if (lane * NO + j < ext.V) op[lane * NO + j] = f2bf(o[j]);
+        continue;
+      }
+      short* op = out + ((long)b * Hq + h0 + g) * DV;
       if (OV > 0) {
 #pragma unroll
         for (int j = 0; j < (OV > 0 ? OV : 1); j++)
           op[lane * OV + j] = f2bf(o[j] * invS);
-      } else if (lane < D) {
+      } else if (lane < DV) {
         op[lane] = f2bf(o[0] * invS);
       }
     }
@@ -388,11 +434,11 @@ torch::Tensor paged_attn_decode(torch::Tensor q, torch::Tensor k_cache,
   TORCH_CHECK(fp8 || k_cache.scalar_type() == torch::kBFloat16,
               "kv cache must be bf16 or fp8_e4m3fn");
 #define LAUNCH_D(DD, CT)                                                        \
-  hipLaunchKernelGGL((paged_decode_kernel<DD, CT>), grid, block, 0, stream,     \
+  hipLaunchKernelGGL((paged_decode_kernel<DD, DD, CT, false>), grid, block, 0, stream, \
                      (const short*)q.data_ptr(), (const CT*)k_cache.data_ptr(), \
                      (const CT*)v_cache.data_ptr(), block_tables.data_ptr<int>(), \
                      seq_lens.data_ptr<int>(), (short*)out.data_ptr(),          \
-                     Hq, Hkv, maxP, G, (float)scale)
+                     Hq, Hkv, maxP, G, (float)scale, DecodeExt{})
   if (D == 128) { if (fp8) LAUNCH_D(128, unsigned char); else LAUNCH_D(128, short); }
   else if (D == 64) { if (fp8) LAUNCH_D(64, unsigned char); else LAUNCH_D(64, short); }
   else if (D == 32) { if (fp8) LAUNCH_D(32, unsigned char); else LAUNCH_D(32, short); }
@@ -400,4 +446,60 @@ torch::Tensor paged_attn_decode(torch::Tensor q, torch::Tensor k_cache,
 #undef LAUNCH_D
   HIP_CHECK_LAST();
   return out;
+}
+
+// General form: key and value widths differ, sliding window with kept first
+// tokens, output turned back by position, strided output rows.
+// q [B, Hq, DK], k_cache [P, 16, Hkv, DK], v_cache [P, Hkv, DV, 16] (bf16),
+// out [B, Hq * V] with any row stride; DK, DV in {32, 64, 128, 256}.
+void paged_attn_decode_window(torch::Tensor q, torch::Tensor k_cache, torch::Tensor v_cache,
+                              torch::Tensor block_tables, torch::Tensor seq_lens,
+                              torch::Tensor out, double scale, long size, long keep,
+                              c10::optional<torch::Tensor> uncs) {
+  TORCH_CHECK(q.is_cuda() && q.scalar_type() == torch::kBFloat16 && q.is_contiguous() && q.dim() == 3);
+  TORCH_CHECK(k_cache.scalar_type() == torch::kBFloat16 && v_cache.scalar_type() == torch::kBFloat16 &&
+              k_cache.is_contiguous() && v_cache.is_contiguous());
+  TORCH_CHECK(block_tables.scalar_type() == torch::kInt && block_tables.is_contiguous() &&
+              seq_lens.scalar_type() == torch::kInt && seq_lens.is_contiguous());
+  const int B = q.size(0), Hq = q.size(1), DK = q.size(2);
+  const int Hkv = k_cache.size(2), DV = v_cache.size(2), maxP = block_tables.size(1);
+  TORCH_CHECK(k_cache.size(1) == 16 && v_cache.size(3) == 16, "page_size must be 16");
+  TORCH_CHECK(k_cache.size(3) == DK && v_cache.size(1) == Hkv && v_cache.size(0) == k_cache.size(0));
+  TORCH_CHECK(Hq % Hkv == 0 && block_tables.size(0) == B && seq_lens.numel() == B);
+  TORCH_CHECK(out.scalar_type() == torch::kBFloat16 && out.size(0) == B && out.stride(1) == 1 &&
+              out.size(1) % Hq == 0);
+  TORCH_CHECK(size > 0 && keep >= 0);
+  const int V = out.size(1) / Hq;
+  TORCH_CHECK(V <= DV);
+  if (uncs.has_value())
+    TORCH_CHECK(uncs->scalar_type() == torch::kFloat32 && uncs->is_contiguous() &&
+                uncs->size(0) == B && uncs->size(1) == V && V % 2 == 0);
+  if (B == 0) return;
+  const int G = Hq / Hkv;
+  DecodeExt e{(int)std::min<long>(size, 1 << 30), (int)std::min<long>(keep, 1 << 30), V,
+              out.stride(0), uncs.has_value() ? uncs->data_ptr<float>() : nullptr, (G + 15) / 16};
+  auto stream = at::hip::getCurrentHIPStream();
+  dim3 grid(B * Hkv * e.gchunks), block(256);
+#define LAUNCH_KV(KK, VV)                                                                  \
+  hipLaunchKernelGGL((paged_decode_kernel<KK, VV, short, true>), grid, block, 0, stream,   \
+                     (const short*)q.data_ptr(), (const short*)k_cache.data_ptr(),         \
+                     (const short*)v_cache.data_ptr(), block_tables.data_ptr<int>(),       \
+                     seq_lens.data_ptr<int>(), (short*)out.data_ptr(), Hq, Hkv, maxP, G,   \
+                     (float)scale, e)
+#define LAUNCH_V(KK)                                                                       \
+  do {                                                                                     \
+    if (DV == 32) LAUNCH_KV(KK, 32);                                                       \
+    else if (DV == 64) LAUNCH_KV(KK, 64);                                                  \
+    else if (DV == 128) LAUNCH_KV(KK, 128);                                                \
+    else if (DV == 256) LAUNCH_KV(KK, 256);                                                \
+    else TORCH_CHECK(false, "unsupported value width ", DV);                               \
+  } while (0)
+  if (DK == 32) LAUNCH_V(32);
+  else if (DK == 64) LAUNCH_V(64);
+  else if (DK == 128) LAUNCH_V(128);
+  else if (DK == 256) LAUNCH_V(256);
+  else TORCH_CHECK(false, "unsupported key width ", DK);
+#undef LAUNCH_V
+#undef LAUNCH_KV
+  HIP_CHECK_LAST();
 }

@@ -1,0 +1,423 @@
+// Attention of prompt portions over the paged KV cache (the new tokens' own
+// keys and values are already in it), so a portion may start anywhere.
+//
+// paged_attn_varlen (bf16, MFMA): one 256-thread workgroup per (sequence,
+// kv-head, 128 query rows).  A "row" is a (token, query head) pair of the
+// kv-head's group, tokens outermost, so grouped heads share every K/V tile and
+// a short portion still fills the 32-row MFMA tiles.  Each of the 4 waves owns
+// 32 rows; KV walks in 64-token tiles (4 pages) double-buffered in LDS.  As in
+// the packed forward kernel, QK^T is computed swapped (S^T = K Q^T), which
+// leaves a row's 64 scores in one lane pair: online softmax without LDS, P
+// repacked to bf16 in registers, O^T = V^T P^T.  V pages are d-major, so a
+// V^T fragment (8 tokens of one d) is one 16-byte copy from page to LDS.
+//
+// Mask: position i sees j if j <= i and (i - j < size or j < keep); tiles
+// between the kept first tokens and the window are never visited.
+//
+// paged_attn_plain (bf16 or float): one wave per (token, head), scalar
+// products in 32-bit; the float32 mode's attention for portions and decoding.
+#include <torch/extension.h>
+#include <ATen/hip/HIPContext.h>
+
+#include "common.h"
+
+typedef __bf16 bf16x8p __attribute__((ext_vector_type(8)));
+
+DEVINL f32x16 mfma32p(bf16x8p a, bf16x8p b, f32x16 c) {
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
+}
+
+DEVINL unsigned pack2p(float lo, float hi) {
+  __hip_bfloat162 h2 = __float22bfloat162_rn(float2{lo, hi});
+  return *reinterpret_cast<unsigned*>(&h2);
+}
+
+struct VarlenArgs {
+  const short* q;        // [T, Hq, DK]
+  const short* kc;       // [P, 16, Hkv, DK]
+  const short* vc;       // [P, Hkv, DV, 16]
+  const int* cu;         // [B + 1] first query token of each sequence
+  const int* seq_lens;   // [B] keys, the portion's own included
+  const int* bt;         // [B, maxP]
+  const float* uncs;     // [T, V] cos | sin or null
+  short* out;            // [T, ldo], head h at columns h * V
+  long ldo;
+  int Hq, Hkv, maxP, V, size, keep;
+  float scale;
+};
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK > 128 || DV > 128) ? 1 : 2)
+void paged_varlen_kernel(VarlenArgs a) {
+  constexpr int NDS = DK / 16, NDT = DV / 32, KV = 64;
+  constexpr int KROW = DK + 8;                 // padded LDS row: spreads the banks
+  constexpr float THR = 11.54f;                // defer-max threshold (log2 units)
+  const int seq = blockIdx.y, kvh = blockIdx.z;
+  const int G = a.Hq / a.Hkv;
+  const int t0 = a.cu[seq], nq = a.cu[seq + 1] - t0;
+  const int L = a.seq_lens[seq];
+  const int start = L - nq;                    // position of the portion's first token
+  const int R = nq * G;
+  const int r0 = blockIdx.x * 128;
+  if (r0 >= R) return;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int col = lane & 31, hi = lane >> 5;
+  const int rw0 = r0 + wid * 32;
+  const bool wave_active = rw0 < R;
+  const int row = min(rw0 + col, R - 1);
+  const bool row_ok = rw0 + col < R;
+  const int tok = row / G, head = kvh * G + row % G;
+  const int qpos = start + tok;
+
+  __shared__ __attribute__((aligned(16))) short Ks[2][KV * KROW];   // [tok][d]
+  __shared__ __attribute__((aligned(16))) short Vs[2][KV * DV];     // [tok/8][d][tok%8]
+
+  bf16x8p qf[NDS];
+  {
+    const short* qr = a.q + ((long)(t0 + tok) * a.Hq + head) * DK;
+#pragma unroll
+    for (int ds = 0; ds < NDS; ds++)
+      qf[ds] = *reinterpret_cast<const bf16x8p*>(qr + 16 * ds + 8 * hi);
+  }
+
+  float m = -INFINITY, sum = 0.f;
+  f32x16 acc[NDT];
+#pragma unroll
+  for (int t = 0; t < NDT; t++) acc[t] = f32x16{};
+
+  // positions covered by the workgroup and by this wave
+  const int pos_lo = start + r0 / G;
+  const int pos_hi = start + min(r0 + 127, R - 1) / G;
+  const int wpos_lo = start + min(rw0, R - 1) / G;
+  const int wpos_hi = start + min(rw0 + 31, R - 1) / G;
+  const int win_tile = max(0, pos_lo - a.size + 1) / KV;
+  const int kept_tiles = min((a.keep + KV - 1) / KV, win_tile);
+  const int ntiles = kept_tiles + pos_hi / KV + 1 - win_tile;
+  const int* btb = a.bt + (long)seq * a.maxP;
+  const int last_page = (L - 1) >> 4;
+
+  constexpr int KCH = KV * DK / 8 / 256;   // 16-byte chunks per thread
+  constexpr int VCH = KV * DV / 8 / 256;
+  s16x8 kr[KCH], vr[VCH];
+  auto tile_of = [&](int it) { return it < kept_tiles ? it : it - kept_tiles + win_tile; };
+  auto load_tile = [&](int tile) {
+#pragma unroll
+    for (int s = 0; s < KCH; s++) {
+      const int c = threadIdx.x + s * 256;
+      const int tk = c / (DK / 8), d0 = (c % (DK / 8)) * 8;
+      const int page = btb[min(tile * 4 + (tk >> 4), last_page)];
+      kr[s] = *reinterpret_cast<const s16x8*>(
+          a.kc + (((long)page * 16 + (tk & 15)) * a.Hkv + kvh) * DK + d0);
+    }
+#pragma unroll
+    for (int s = 0; s < VCH; s++) {
+      const int c = threadIdx.x + s * 256;        // (page, d, half) fastest last
+      const int half = c & 1, d = (c >> 1) % DV, pg = (c >> 1) / DV;
+      const int page = btb[min(tile * 4 + pg, last_page)];
+      vr[s] = *reinterpret_cast<const s16x8*>(
+          a.vc + (((long)page * a.Hkv + kvh) * DV + d) * 16 + half * 8);
+    }
+  };
+  auto store_tile = [&](int buf) {
+#pragma unroll
+    for (int s = 0; s < KCH; s++) {
+      const int c = threadIdx.x + s * 256;
+      const int tk = c / (DK / 8), d0 = (c % (DK / 8)) * 8;
+      *reinterpret_cast<s16x8*>(&Ks[buf][tk * KROW + d0]) = kr[s];
+    }
+#pragma unroll
+    for (int s = 0; s < VCH; s++) {
+      const int c = threadIdx.x + s * 256;
+      const int half = c & 1, d = (c >> 1) % DV, pg = (c >> 1) / DV;
+      *reinterpret_cast<s16x8*>(&Vs[buf][((pg * 2 + half) * DV + d) * 8]) = vr[s];
+    }
+  };
+
+  load_tile(tile_of(0));
+  for (int it = 0; it < ntiles; it++) {
+    const int buf = it & 1, kv0 = tile_of(it) * KV;
+    store_tile(buf);          // readers of `buf` passed the previous barrier
+    __syncthreads();
+    if (it + 1 < ntiles) load_tile(tile_of(it + 1));
+    // whole tile invisible to this wave?
+    if (!wave_active || kv0 > wpos_hi ||
+        (wpos_lo - (kv0 + KV - 1) >= a.size && kv0 >= a.keep))
+      continue;
+
+    f32x16 st[2];
+#pragma unroll
+    for (int sub = 0; sub < 2; sub++) {
+      st[sub] = f32x16{};
+#pragma unroll
+      for (int ds = 0; ds < NDS; ds++) {
+        const bf16x8p kf = *reinterpret_cast<const bf16x8p*>(
+            &Ks[buf][(sub * 32 + col) * KROW + 16 * ds + 8 * hi]);
+        st[sub] = mfma32p(kf, qf[ds], st[sub]);
+      }
+    }
+    const float sl2 = a.scale * 1.4426950408889634f;
+    const bool full = kv0 + KV - 1 <= wpos_lo &&
+                      (wpos_hi - kv0 < a.size || kv0 + KV <= a.keep);
+    float p[32];
+#pragma unroll
+    for (int i = 0; i < 32; i++) {
+      const int r = i & 15;
+      const int ki = kv0 + 32 * (i >> 4) + (r & 3) + 8 * (r >> 2) + 4 * hi;
+      const float s = st[i >> 4][r] * sl2;
+      p[i] = (full || (ki <= qpos && (qpos - ki < a.size || ki < a.keep))) ? s : -INFINITY;
+    }
+    float pmax = p[0];
+#pragma unroll
+    for (int i = 1; i < 32; i++) pmax = fmaxf(pmax, p[i]);
+    pmax = fmaxf(pmax, __shfl_xor(pmax, 32));
+    float alpha = 1.f;
+    const bool need = !(pmax - m <= THR);      // also true while m is -inf
+    if (__any(need)) {
+      const float mn = fmaxf(m, pmax);
+      alpha = (m == -INFINITY) ? 0.f : exp2f(m - mn);
+      m = mn;
+#pragma unroll
+      for (int t = 0; t < NDT; t++)
+#pragma unroll
+        for (int r = 0; r < 16; r++) acc[t][r] *= alpha;
+    }
+    float rs = 0.f;
+#pragma unroll
+    for (int i = 0; i < 32; i++) {
+      p[i] = (p[i] > -INFINITY) ? exp2f(p[i] - m) : 0.f;
+      rs += p[i];
+    }
+    rs += __shfl_xor(rs, 32);
+    sum = sum * alpha + rs;
+    // P^T fragments: lane holds P[row][16 ks + 8 hi + j]
+    bf16x8p pf[4];
+#pragma unroll
+    for (int ks = 0; ks < 4; ks++) {
+      const int b0 = ks * 8;
+      const unsigned w01 = pack2p(p[b0 + 0], p[b0 + 1]);
+      const unsigned w23 = pack2p(p[b0 + 2], p[b0 + 3]);
+      const unsigned w45 = pack2p(p[b0 + 4], p[b0 + 5]);
+      const unsigned w67 = pack2p(p[b0 + 6], p[b0 + 7]);
+      auto rA = __builtin_amdgcn_permlane32_swap(w01, w45, false, false);
+      auto rB = __builtin_amdgcn_permlane32_swap(w23, w67, false, false);
+      union { unsigned u[4]; bf16x8p f; } fr;
+      fr.u[0] = (unsigned)rA[0];
+      fr.u[1] = (unsigned)rB[0];
+      fr.u[2] = (unsigned)rA[1];
+      fr.u[3] = (unsigned)rB[1];
+      pf[ks] = fr.f;
+    }
+#pragma unroll
+    for (int t = 0; t < NDT; t++)
+#pragma unroll
+      for (int ks = 0; ks < 4; ks++) {
+        const bf16x8p vf = *reinterpret_cast<const bf16x8p*>(
+            &Vs[buf][((2 * ks + hi) * DV + t * 32 + col) * 8]);
+        acc[t] = mfma32p(vf, pf[ks], acc[t]);
+      }
+  }
+
+  if (!wave_active || !row_ok) return;
+  const float inv = sum > 0.f ? 1.f / sum : 0.f;
+  short* op = a.out + (long)(t0 + tok) * a.ldo + (long)head * a.V;
+  const float* cs = a.uncs ? a.uncs + (long)(t0 + tok) * a.V : nullptr;
+  const int half = a.V / 2;
+  const bool wide = (a.V & 3) == 0 && (a.ldo & 3) == 0 && ((size_t)a.out & 7) == 0;
+#pragma unroll
+  for (int t = 0; t < NDT; t++)
+#pragma unroll
+    for (int g = 0; g < 4; g++) {
+      const int d0 = t * 32 + 8 * g + 4 * hi;   // registers 4g..4g+3 are d0..d0+3
+      if (d0 >= a.V) continue;
+      float o[4];
+#pragma unroll
+      for (int j = 0; j < 4; j++) o[j] = acc[t][4 * g + j] * inv;
+      if (cs) {
+#pragma unroll
+        for (int j = 0; j < 4; j += 2) {
+          const int pr = min((d0 + j) >> 1, half - 1);
+          const float c = cs[pr], s = cs[half + pr], u = o[j], v = o[j + 1];
+          o[j] = u * c + v * s;
+          o[j + 1] = v * c - u * s;
+        }
+      }
+      if (wide)
+        stv<4>(op + d0, o);
+      else
+#pragma unroll
+        for (int j = 0; j < 4; j++)
+          if (d0 + j < a.V) stf(op + d0 + j, o[j]);
+    }
+}
+
+// -------------------------------------------------------- plain, any type
+template <typename T>
+__global__ __launch_bounds__(256) void paged_plain_kernel(
+    const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc,
+    const int* __restrict__ row_seq, const long* __restrict__ positions,
+    const int* __restrict__ bt, const float* __restrict__ uncs, T* __restrict__ out,
+    long rows, int Hq, int Hkv, int DK, int DV, int V, int maxP, long ldo, int size, int keep,
+    float scale) {
+  __shared__ float qs[4][256], ps[4][64], os[4][256];
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const long unit = blockIdx.x * 4L + w;
+  if (unit >= rows * Hq) return;
+  const long t = unit / Hq;
+  const int h = (int)(unit % Hq), kvh = h / (Hq / Hkv);
+  const int pos = (int)positions[t];
+  const int* btb = bt + (long)row_seq[t] * maxP;
+  for (int d = lane; d < DK; d += 64) qs[w][d] = ldf(q + (t * Hq + h) * (long)DK + d);
+  lds_fence_wave_kv();
+  float m = -INFINITY, sum = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
+  const int win_tile = max(0, pos - size + 1) / 64;
+  const int kept = min((keep + 63) / 64, win_tile);
+  const int n = kept + pos / 64 + 1 - win_tile;
+  for (int it = 0; it < n; it++) {
+    const int k0 = (it < kept ? it : it - kept + win_tile) * 64;
+    const int ki = k0 + lane;
+    float s = -INFINITY;
+    if (ki <= pos && (pos - ki < size || ki < keep)) {
+      const T* kr = kc + (((long)btb[min(ki >> 4, maxP - 1)] * 16 + (ki & 15)) * Hkv + kvh) * DK;
+      float d0 = 0.f;
+      for (int d = 0; d < DK; d += 4) {
+        float v[4];
+        ldv<4>(kr + d, v);
+#pragma unroll
+        for (int j = 0; j < 4; j++) d0 += v[j] * qs[w][d + j];
+      }
+      s = d0 * scale;
+    }
+    const float mn = fmaxf(m, wave_max(s));
+    const float alpha = (m == -INFINITY) ? 0.f : expf(m - mn);
+    const float p = (s == -INFINITY) ? 0.f : expf(s - mn);
+    m = mn;
+    sum = sum * alpha + wave_sum(p);
+    ps[w][lane] = p;
+    lds_fence_wave_kv();
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      const int d = lane + 64 * r;
+      acc[r] *= alpha;
+      if (d >= V) continue;
+      for (int pg = 0; pg < 4; pg++) {
+        if (k0 + 16 * pg > pos) break;
+        const T* vr = vc + (((long)btb[min((k0 >> 4) + pg, maxP - 1)] * Hkv + kvh) * DV + d) * 16;
+        for (int j = 0; j < 16; j++) acc[r] += ps[w][16 * pg + j] * ldf(vr + j);
+      }
+    }
+    lds_fence_wave_kv();
+  }
+#pragma unroll
+  for (int r = 0; r < 4; r++)
+    if (lane + 64 * r < V) os[w][lane + 64 * r] = acc[r] / sum;
+  lds_fence_wave_kv();
+  T* op = out + t * ldo + (long)h * V;
+  const int half = V / 2;
+  for (int d = lane; d < V; d += 64) {
+    float o = os[w][d];
+    if (uncs) {
+      const float c = uncs[t * V + (d >> 1)], s = uncs[t * V + half + (d >> 1)];
+      o = o * c + ((d & 1) ? -os[w][d ^ 1] : os[w][d ^ 1]) * s;
+    }
+    stf(op + d, o);
+  }
+}
+
+// ======================================================== host wrappers ==
+static void check_cache(const torch::Tensor& q, const torch::Tensor& kc, const torch::Tensor& vc,
+                        const torch::Tensor& bt, const torch::Tensor& out,
+                        const c10::optional<torch::Tensor>& uncs, long size, long keep) {
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous());
+  TORCH_CHECK(kc.is_contiguous() && vc.is_contiguous() && kc.dim() == 4 && vc.dim() == 4);
+  TORCH_CHECK(kc.scalar_type() == q.scalar_type() && vc.scalar_type() == q.scalar_type() &&
+              out.scalar_type() == q.scalar_type(), "q, cache and output of one type");
+  TORCH_CHECK(kc.size(1) == 16 && vc.size(3) == 16, "page_size must be 16");
+  TORCH_CHECK(kc.size(3) == q.size(2) && vc.size(1) == kc.size(2) && vc.size(0) == kc.size(0));
+  TORCH_CHECK(q.size(1) % kc.size(2) == 0);
+  TORCH_CHECK(bt.scalar_type() == torch::kInt && bt.is_contiguous() && bt.dim() == 2 && bt.size(1) > 0);
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == q.size(0) && out.stride(1) == 1 &&
+              out.size(1) % q.size(1) == 0 && out.size(1) / q.size(1) <= vc.size(2));
+  TORCH_CHECK(size > 0 && keep >= 0);
+  if (uncs.has_value())
+    TORCH_CHECK(uncs->scalar_type() == torch::kFloat32 && uncs->is_contiguous() &&
+                uncs->size(0) == q.size(0) && uncs->size(1) * q.size(1) == out.size(1) &&
+                uncs->size(1) % 2 == 0);
+}
+
+void paged_attn_varlen(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor cu,
+                       torch::Tensor seq_lens, torch::Tensor bt, torch::Tensor out, long max_q,
+                       double scale, long size, long keep, c10::optional<torch::Tensor> uncs) {
+  check_cache(q, kc, vc, bt, out, uncs, size, keep);
+  TORCH_CHECK(q.scalar_type() == torch::kBFloat16);
+  const int B = seq_lens.numel();
+  TORCH_CHECK(cu.scalar_type() == torch::kInt && cu.is_contiguous() && cu.numel() == B + 1 &&
+              seq_lens.scalar_type() == torch::kInt && seq_lens.is_contiguous() && bt.size(0) == B);
+  if (B == 0 || q.size(0) == 0) return;
+  VarlenArgs a;
+  a.q = (const short*)q.data_ptr();
+  a.kc = (const short*)kc.data_ptr();
+  a.vc = (const short*)vc.data_ptr();
+  a.cu = cu.data_ptr<int>();
+  a.seq_lens = seq_lens.data_ptr<int>();
+  a.bt = bt.data_ptr<int>();
+  a.uncs = uncs.has_value() ? uncs->data_ptr<float>() : nullptr;
+  a.out = (short*)out.data_ptr();
+  a.ldo = out.stride(0);
+  a.Hq = q.size(1);
+  a.Hkv = kc.size(2);
+  a.maxP = bt.size(1);
+  a.V = out.size(1) / q.size(1);
+  a.size = (int)std::min<long>(size, 1 << 30);
+  a.keep = (int)std::min<long>(keep, 1 << 30);
+  a.scale = scale;
+  const int DK = q.size(2), DV = vc.size(2);
+  dim3 grid((max_q * (a.Hq / a.Hkv) + 127) / 128, B, a.Hkv);
+  auto stream = at::hip::getCurrentHIPStream();
+#define LAUNCH(KK, VV) \
+  hipLaunchKernelGGL((paged_varlen_kernel<KK, VV>), grid, dim3(256), 0, stream, a)
+#define LAUNCH_V(KK)                                              \
+  do {                                                            \
+    if (DV == 32) LAUNCH(KK, 32);                                 \
+    else if (DV == 64) LAUNCH(KK, 64);                            \
+    else if (DV == 128) LAUNCH(KK, 128);                          \
+    else if (DV == 256) LAUNCH(KK, 256);                          \
+    else TORCH_CHECK(false, "unsupported value width ", DV);      \
+  } while (0)
+  if (DK == 32) LAUNCH_V(32);
+  else if (DK == 64) LAUNCH_V(64);
+  else if (DK == 128) LAUNCH_V(128);
+  else if (DK == 256) LAUNCH_V(256);
+  else TORCH_CHECK(false, "unsupported key width ", DK);
+#undef LAUNCH_V
+#undef LAUNCH
+  HIP_CHECK_LAST();
+}
+
+void paged_attn_plain(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor row_seq,
+                      torch::Tensor positions, torch::Tensor bt, torch::Tensor out, double scale,
+                      long size, long keep, c10::optional<torch::Tensor> uncs) {
+  check_cache(q, kc, vc, bt, out, uncs, size, keep);
+  const long rows = q.size(0);
+  TORCH_CHECK(row_seq.scalar_type() == torch::kInt && row_seq.is_contiguous() && row_seq.numel() == rows);
+  TORCH_CHECK(positions.scalar_type() == torch::kLong && positions.is_contiguous() && positions.numel() == rows);
+  const int DK = q.size(2), DV = vc.size(2), V = out.size(1) / q.size(1);
+  TORCH_CHECK(DK <= 256 && DV <= 256 && DK % 4 == 0);
+  if (rows == 0) return;
+  const long units = rows * q.size(1);
+  auto stream = at::hip::getCurrentHIPStream();
+#define LAUNCH(TT)                                                                            \
+  hipLaunchKernelGGL((paged_plain_kernel<TT>), dim3((units + 3) / 4), dim3(256), 0, stream,   \
+                     (const TT*)q.data_ptr(), (const TT*)kc.data_ptr(), (const TT*)vc.data_ptr(), \
+                     row_seq.data_ptr<int>(), positions.data_ptr<long>(), bt.data_ptr<int>(), \
+                     uncs.has_value() ? uncs->data_ptr<float>() : nullptr, (TT*)out.data_ptr(), \
+                     rows, (int)q.size(1), (int)kc.size(2), DK, DV, V, (int)bt.size(1),        \
+                     out.stride(0), (int)std::min<long>(size, 1 << 30),                        \
+                     (int)std::min<long>(keep, 1 << 30), (float)scale)
+  if (q.scalar_type() == torch::kBFloat16) LAUNCH(short);
+  else {
+    TORCH_CHECK(q.scalar_type() == torch::kFloat32);
+    LAUNCH(float);
+  }
+#undef LAUNCH
+  HIP_CHECK_LAST();
+}

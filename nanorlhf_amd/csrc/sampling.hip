@@ -1,4 +1,4 @@
-// Temperature / top-p token sampling over [B, V] bf16 logits.
+// Temperature / top-p token sampling over [B, V] bf16 or float32 logits.
 // One 256-thread workgroup per row, four vectorized passes (s16x8 16-B
 // loads — the scalar version measured 2.7 ms/row-batch, ~6x off BW):
 //   1. fused online (max, exp-sum) + argmax
@@ -25,7 +25,8 @@ DEVINL float warp_incl_scan(float v, int lane) {
   return v;
 }
 
-__global__ void sample_topp_kernel(const short* __restrict__ logits,
+template <typename LT>
+__global__ void sample_topp_kernel(const LT* __restrict__ logits,
                                    long* __restrict__ out,
                                    float* __restrict__ out_lp,  // nullable
                                    int V, float temperature, float top_p,
@@ -40,7 +41,7 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
   __shared__ int found_sh;
   __shared__ float wsum[SBLOCK / 64];
   const long row = blockIdx.x;
-  const short* lr = logits + row * (long)V;
+  const LT* lr = logits + row * (long)V;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int nvec = V / 8;
 
@@ -53,15 +54,16 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
   int am = 0;
   const float invT = temperature > 0.f ? 1.f / temperature : 1.f;
   for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-    s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+    float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
     for (int j = 0; j < 8; j++) {
-      const float l = bf2f(v[j]);
+      const float l = v[j];
       if (l > lmax) { lmax = l; am = i * 8 + j; }
     }
   }
   for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK) {
-    const float l = bf2f(lr[i]);
+    const float l = ldf(lr + i);
     if (l > lmax) { lmax = l; am = i; }
   }
   {  // merge argmax across the block
@@ -89,16 +91,17 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
       float se = 0.f;
       const float M1 = wm_[0];
       for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-        s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+        float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
-        for (int j = 0; j < 8; j++) se += __expf(bf2f(v[j]) - M1);
+        for (int j = 0; j < 8; j++) se += __expf(v[j] - M1);
       }
       for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK)
-        se += __expf(bf2f(lr[i]) - M1);
+        se += __expf(ldf(lr + i) - M1);
       se = block_sum<SBLOCK>(se, sm);
       if (threadIdx.x == 0) {
         out[row] = argmax_sh;
-        out_lp[row] = bf2f(lr[argmax_sh]) - (M1 + __logf(se));
+        out_lp[row] = ldf(lr + argmax_sh) - (M1 + __logf(se));
       }
     } else if (threadIdx.x == 0) {
       out[row] = argmax_sh;
@@ -125,10 +128,11 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
 #pragma unroll
     for (int b = 0; b < 32; b++) hb[b] = 0.f;
     for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+      float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
       for (int j = 0; j < 8; j++) {
-        const float u = bf2f(v[j]) * invT - M;
+        const float u = v[j] * invT - M;
         const float e = __expf(u);
         sacc += e;
         int b = (int)(u + URANGE);
@@ -137,7 +141,7 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
       }
     }
     for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK) {
-      const float u = bf2f(lr[i]) * invT - M;
+      const float u = ldf(lr + i) * invT - M;
       const float e = __expf(u);
       sacc += e;
       int b = (int)(u + URANGE);
@@ -186,10 +190,11 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
     for (int b = 0; b < 32; b++) hb[b] = 0.f;
     const float sub = 32.0f / span;
     for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+      float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
       for (int j = 0; j < 8; j++) {
-        const float u = bf2f(v[j]) * invT - M;
+        const float u = v[j] * invT - M;
         if (u >= lo && u < lo + span) {
           int b = (int)((u - lo) * sub);
           b = max(0, min(31, b));
@@ -198,7 +203,7 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
       }
     }
     for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK) {
-      const float u = bf2f(lr[i]) * invT - M;
+      const float u = ldf(lr + i) * invT - M;
       if (u >= lo && u < lo + span) {
         int b = (int)((u - lo) * sub);
         b = max(0, min(31, b));
@@ -241,15 +246,16 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
   // ---- pass 4: per-thread kept mass + block scan + owner walk ----------
   float own = 0.f;
   for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-    s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+    float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
     for (int j = 0; j < 8; j++) {
-      const float u = bf2f(v[j]) * invT - M;
+      const float u = v[j] * invT - M;
       if (u >= u_thresh) own += __expf(u);
     }
   }
   for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK) {
-    const float u = bf2f(lr[i]) * invT - M;
+    const float u = ldf(lr + i) * invT - M;
     if (u >= u_thresh) own += __expf(u);
   }
   float incl = warp_incl_scan(own, lane);
@@ -273,10 +279,11 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
     float acc = excl;
     int found = -1;
     for (int i = threadIdx.x; i < nvec; i += SBLOCK) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(lr + i * 8);
+      float v[8];
+      ldv<8>(lr + i * 8, v);
 #pragma unroll
       for (int j = 0; j < 8; j++) {
-        const float u = bf2f(v[j]) * invT - M;
+        const float u = v[j] * invT - M;
         if (u >= u_thresh) {
           acc += __expf(u);
           if (target < acc && found < 0) found = i * 8 + j;
@@ -284,7 +291,7 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
       }
     }
     for (int i = nvec * 8 + threadIdx.x; i < V; i += SBLOCK) {
-      const float u = bf2f(lr[i]) * invT - M;
+      const float u = ldf(lr + i) * invT - M;
       if (u >= u_thresh) {
         acc += __expf(u);
         if (target < acc && found < 0) found = i;
@@ -298,23 +305,27 @@ __global__ void sample_topp_kernel(const short* __restrict__ logits,
     out[row] = f;
     // logprob of the chosen token under the temperature-scaled softmax
     // (matches the scoring pass's logits/temperature quirk, grpo_trainer.py:547)
-    if (out_lp) out_lp[row] = bf2f(lr[f]) * invT - (M + __logf(S));
+    if (out_lp) out_lp[row] = ldf(lr + f) * invT - (M + __logf(S));
   }
 }
 
 torch::Tensor sample_topp(torch::Tensor logits, double temperature, double top_p,
                           long seed, long step) {
   TORCH_CHECK(logits.dim() == 2 && logits.is_contiguous());
-  TORCH_CHECK(logits.scalar_type() == torch::kBFloat16, "sample_topp expects bf16 logits");
+  const bool half = logits.scalar_type() == torch::kBFloat16;
+  TORCH_CHECK(half || logits.scalar_type() == torch::kFloat32, "logits must be bf16 or float32");
   const long B = logits.size(0);
   const int V = logits.size(1);
   auto out = torch::empty({B}, logits.options().dtype(torch::kLong));
   if (B == 0) return out;
   auto stream = at::hip::getCurrentHIPStream();
-  hipLaunchKernelGGL(sample_topp_kernel, dim3(B), dim3(SBLOCK), 0, stream,
-                     (const short*)logits.data_ptr(), out.data_ptr<long>(), nullptr,
-                     V, (float)temperature, (float)top_p,
-                     (unsigned long long)seed, (unsigned long long)step, nullptr);
+#define LAUNCH(LT)                                                              \
+  hipLaunchKernelGGL(sample_topp_kernel<LT>, dim3(B), dim3(SBLOCK), 0, stream,  \
+                     (const LT*)logits.data_ptr(), out.data_ptr<long>(),        \
+                     nullptr, V, (float)temperature, (float)top_p,            \
+                     (unsigned long long)seed, (unsigned long long)step, nullptr)
+  if (half) LAUNCH(short); else LAUNCH(float);
+#undef LAUNCH
   HIP_CHECK_LAST();
   return out;
 }
@@ -325,7 +336,8 @@ std::vector<torch::Tensor> sample_topp_dev(torch::Tensor logits, double temperat
   // hipGraph capture/replay (the immediate-arg form would freeze the step).
   // Also returns the chosen token's logprob (vLLM logprobs parity).
   TORCH_CHECK(logits.dim() == 2 && logits.is_contiguous());
-  TORCH_CHECK(logits.scalar_type() == torch::kBFloat16);
+  const bool half = logits.scalar_type() == torch::kBFloat16;
+  TORCH_CHECK(half || logits.scalar_type() == torch::kFloat32, "logits must be bf16 or float32");
   TORCH_CHECK(step.scalar_type() == torch::kLong && step.is_cuda());
   const long B = logits.size(0);
   const int V = logits.size(1);
@@ -333,11 +345,13 @@ std::vector<torch::Tensor> sample_topp_dev(torch::Tensor logits, double temperat
   auto lp = torch::empty({B}, logits.options().dtype(torch::kFloat32));
   if (B == 0) return {out, lp};
   auto stream = at::hip::getCurrentHIPStream();
-  hipLaunchKernelGGL(sample_topp_kernel, dim3(B), dim3(SBLOCK), 0, stream,
-                     (const short*)logits.data_ptr(), out.data_ptr<long>(),
-                     lp.data_ptr<float>(), V,
-                     (float)temperature, (float)top_p,
-                     (unsigned long long)seed, 0ull, step.data_ptr<long>());
+#define LAUNCH(LT)                                                              \
+  hipLaunchKernelGGL(sample_topp_kernel<LT>, dim3(B), dim3(SBLOCK), 0, stream,  \
+                     (const LT*)logits.data_ptr(), out.data_ptr<long>(),        \
+                     lp.data_ptr<float>(), V, (float)temperature, (float)top_p,            \
+                     (unsigned long long)seed, 0ull, step.data_ptr<long>())
+  if (half) LAUNCH(short); else LAUNCH(float);
+#undef LAUNCH
   HIP_CHECK_LAST();
   return {out, lp};
 }

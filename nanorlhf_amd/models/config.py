@@ -10,6 +10,22 @@ from __future__ import annotations
 from dataclasses import dataclass, field, asdict
 
 
+@dataclass(frozen=True)
+class KVSpec:
+    """A layer that caches keys and values of every token, in pages."""
+    heads: int
+    k_dim: int     # cached widths (already padded to what the kernels tile)
+    v_dim: int
+
+
+@dataclass(frozen=True)
+class StateSpec:
+    """A layer that keeps one 32-bit matrix per head and sequence, in a slot."""
+    heads: int
+    dim: int
+    vdim: int
+
+
 @dataclass
 class ModelConfig:
     vocab_size: int = 151936
@@ -29,12 +45,32 @@ class ModelConfig:
     bidirectional: bool = False
     num_labels: int = 0  # >0 adds a classification/score head
 
+    def cache_layers(self) -> list:
+        """What each layer keeps of a sequence (KVSpec or StateSpec)."""
+        return [KVSpec(self.num_kv_heads, self.head_dim, self.head_dim)] * self.num_layers
+
     def to_dict(self):
         return asdict(self)
 
     @staticmethod
     def from_dict(d):
         return ModelConfig(**d)
+
+
+def _gonurax_layers(n, *, heads, dim, vdim, attn_heads, kv_heads, attn_dim, ff, window,
+                    keep_first) -> dict:
+    """n layers, retention / attention / lightning in turn, of equal sizes."""
+    decay = [1.0 - 2.0 ** -(5 + 7 * h / max(heads - 1, 1)) for h in range(heads)]
+    linear = dict(heads=heads, dim=dim, vdim=vdim, decay=decay)
+    kinds = [
+        ("retention", dict(linear, rot=dict(dims=dim, base=10000.0))),
+        ("attention", dict(heads=attn_heads, kv_heads=kv_heads, dim=attn_dim, vdim=attn_dim,
+                           rot=dict(dims=attn_dim, base=500000.0), scale=attn_dim ** -0.5,
+                           mask=dict(size=window, keep_first=keep_first))),
+        ("lightning", dict(linear)),
+    ]
+    return dict(layers=[dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1],
+                             mlp=dict(kind="dense", ff=ff)) for i in range(n)])
 
 
 PRESETS: dict[str, dict] = {
@@ -58,6 +94,18 @@ PRESETS: dict[str, dict] = {
                      intermediate_size=4096, bidirectional=True, num_labels=1,
                      rope_theta=1e4, max_position=4096, tie_word_embeddings=False,
                      qkv_bias=True),
+    # Gonurax shapes (random-init): retention, windowed attention and lightning
+    # layers in turn.  "-1.5b" has the width and feed-forward of qwen2.5-1.5b.
+    "gonurax-tiny": dict(architecture="Gonurax", dtype="float32", vocab_size=1024,
+                         hidden_size=128, norm_groups=4, residual_mult=0.5,
+                         **_gonurax_layers(4, heads=2, dim=32, vdim=48, attn_heads=4,
+                                           kv_heads=2, attn_dim=32, ff=192, window=24,
+                                           keep_first=3)),
+    "gonurax-1.5b": dict(architecture="Gonurax", vocab_size=151936, hidden_size=1536,
+                         norm_groups=4, residual_mult=0.5,
+                         **_gonurax_layers(28, heads=12, dim=128, vdim=128, attn_heads=12,
+                                           kv_heads=2, attn_dim=128, ff=8960, window=1024,
+                                           keep_first=4)),
     # tiny reward encoder for CPU tests
     "rm-tiny": dict(vocab_size=1024, hidden_size=128, num_layers=2, num_heads=4,
                     num_kv_heads=4, head_dim=32, intermediate_size=512,
@@ -66,9 +114,14 @@ PRESETS: dict[str, dict] = {
 }
 
 
-def get_config(name: str, **overrides) -> ModelConfig:
+def get_config(name: str, **overrides):
+    """The preset's configuration: a ModelConfig, or the configuration class
+    of the architecture the preset names (models/registry.py)."""
     if name not in PRESETS:
         raise KeyError(f"unknown model preset {name!r}; have {sorted(PRESETS)}")
     d = dict(PRESETS[name])
     d.update(overrides)
+    if "architecture" in d:
+        from .registry import config_class
+        return config_class(d.pop("architecture"))(**d)
     return ModelConfig(**d)

@@ -14,8 +14,8 @@ Replaces the reference's transformers Qwen2 + flash_attention_2 stack
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Optional
+from dataclasses import dataclass, field
+from typing import Callable, Optional
 
 import torch
 import torch.nn as nn
@@ -26,9 +26,28 @@ from .config import ModelConfig, get_config
 
 
 @dataclass
+class Portions:
+    """The multi-token entries of an engine step, packed; every tensor is on
+    the model's device and int32."""
+    cu: torch.Tensor               # [B+1] first row of each portion
+    seq_lens: torch.Tensor         # [B] tokens of the sequence, these included
+    block_tables: torch.Tensor     # [B, P]
+    row_seq: torch.Tensor          # [rows] portion of each row
+    state_slots: torch.Tensor      # [B]
+    fresh: torch.Tensor            # [B] 1 where the portion starts its sequence
+    chunks: torch.Tensor           # [3, n] portion, first row, tokens (<= 64)
+    chunk_first: torch.Tensor      # [B+1] first chunk of each portion
+    max_q: int = 0                 # longest portion
+
+
+@dataclass
 class AttnContext:
-    """Per-forward attention routing info."""
-    mode: str                      # "train" | "prefill" | "decode"
+    """Per-forward attention routing info.
+
+    "train" and "prefill" pack whole sequences (cu_seqlens); "decode" is one
+    token of each sequence; "step" is one batch of n_decode single tokens
+    followed by the tokens of `portions`, all over the cache."""
+    mode: str                      # "train" | "prefill" | "decode" | "step"
     positions: torch.Tensor        # [T] int64 position ids
     cu_seqlens: Optional[torch.Tensor] = None   # [B+1] int32 (train/prefill)
     max_seqlen: int = 0
@@ -37,7 +56,22 @@ class AttnContext:
     slots: Optional[torch.Tensor] = None        # [T] int64 flat slot ids
     block_tables: Optional[torch.Tensor] = None  # [B, P] int32 (decode)
     seq_lens: Optional[torch.Tensor] = None      # [B] int32 (decode)
+    state_slots: Optional[torch.Tensor] = None   # [B] int32 (decode)
     causal: bool = True
+    portions: Optional[Portions] = None
+    on_layer: Optional[Callable] = None          # observer: (layer, residual stream)
+    _angles: dict = field(default_factory=dict)
+
+    @property
+    def n_decode(self) -> int:
+        """Single-token rows at the head of a "step" or "decode" batch."""
+        return 0 if self.seq_lens is None else self.seq_lens.shape[0]
+
+    def angles(self, rotation) -> torch.Tensor:
+        """cos | sin rows of this batch's tokens, once per distinct rotation."""
+        if rotation.key not in self._angles:
+            self._angles[rotation.key] = rotation.angles(self.positions)
+        return self._angles[rotation.key]
 
 
 def dtype_of(cfg: ModelConfig):
@@ -71,13 +105,16 @@ class Attention(nn.Module):
         q = ops.rope_apply(q, rope_table, ctx.positions)
         k = ops.rope_apply(k, rope_table, ctx.positions)
 
-        if ctx.mode in ("prefill", "decode") and ctx.kv_caches is not None:
+        if ctx.mode != "train" and ctx.kv_caches is not None:
             k_cache, v_cache = ctx.kv_caches[self.layer_idx]
             ops.kv_append(k, v, ctx.slots, k_cache, v_cache)
 
         if ctx.mode == "decode":
             o = ops.paged_attn_decode(q, *ctx.kv_caches[self.layer_idx],
                                       ctx.block_tables, ctx.seq_lens, self.scale)
+        elif ctx.mode == "step":
+            o = torch.empty(T, self.q_size, dtype=q.dtype, device=q.device)
+            ops.paged_attn(q, *ctx.kv_caches[self.layer_idx], ctx, o, self.scale)
         else:
             o = ops.flash_attn_varlen(q, k, v, ctx.cu_seqlens, ctx.max_seqlen,
                                       self.scale, causal=ctx.causal)
@@ -154,6 +191,10 @@ class Transformer(nn.Module):
 
 
 class CausalLM(nn.Module):
+    extensions = ("_C", "_serve")       # HIP extensions its forward needs
+    kv_cache_dtypes = ("fp8_e4m3", "bf16")
+    packed_prefill = True               # whole prompts run without reading the cache
+
     def __init__(self, cfg: ModelConfig):
         super().__init__()
         self.cfg = cfg

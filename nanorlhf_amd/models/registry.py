@@ -1,0 +1,70 @@
+"""Model architectures by the name a checkpoint's config.json gives them."""
+from __future__ import annotations
+
+import json
+import os
+from dataclasses import dataclass
+from typing import Callable
+
+import torch
+
+from .config import ModelConfig
+from .gonurax import GonuraxConfig, GonuraxLM
+from .hf_import import load_hf_tensors, load_pretrained
+from .qwen2 import CausalLM
+
+
+def _load_gonurax(path: str, dtype: str | None = None, **overrides) -> GonuraxLM:
+    cfg = GonuraxConfig.from_json(read_config(path), **({"dtype": dtype} if dtype else {}),
+                                  **overrides)
+    model = GonuraxLM(cfg).to(getattr(torch, cfg.dtype))
+    model.load(load_hf_tensors(path))
+    return model
+
+
+@dataclass(frozen=True)
+class Architecture:
+    config: type
+    model: type
+    load: Callable        # (path, dtype=None, **config overrides) -> model
+
+
+ARCHITECTURES = {
+    "Qwen2ForCausalLM": Architecture(ModelConfig, CausalLM, load_pretrained),
+    "Gonurax": Architecture(GonuraxConfig, GonuraxLM, _load_gonurax),
+}
+
+
+def read_config(path: str) -> dict:
+    with open(os.path.join(path, "config.json")) as f:
+        return json.load(f)
+
+
+def architecture_of(path: str) -> Architecture:
+    """By "architecture", or the first known of "architectures"; a config
+    that names none is taken for Qwen2, as before."""
+    c = read_config(path)
+    names = [c["architecture"]] if "architecture" in c else c.get("architectures") or []
+    for n in names:
+        if n in ARCHITECTURES:
+            return ARCHITECTURES[n]
+    if not names or any("Qwen2" in n for n in names):
+        return ARCHITECTURES["Qwen2ForCausalLM"]
+    raise ValueError(f"unsupported architecture {names}; have {sorted(ARCHITECTURES)}")
+
+
+def config_class(name: str) -> type:
+    return ARCHITECTURES[name].config
+
+
+def build_model(cfg):
+    """A randomly initialised model of a configuration."""
+    for a in ARCHITECTURES.values():
+        if type(cfg) is a.config:
+            return a.model(cfg)
+    raise TypeError(f"no model for {type(cfg).__name__}")
+
+
+def load_model(path: str, dtype: str | None = None, **overrides):
+    """The model of a checkpoint folder (config.json and *.safetensors)."""
+    return architecture_of(path).load(path, dtype=dtype, **overrides)

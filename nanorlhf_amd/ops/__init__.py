@@ -2,8 +2,10 @@
 
 Every hot op has two paths:
   * GPU (``tensor.is_cuda``): the hand-written gfx950 HIP kernel from the
-    in-tree extension ``nanorlhf_amd/_C.so``.  If the extension is missing on
-    a machine with a GPU this raises loudly — there is NO silent eager
+    in-tree extensions ``nanorlhf_amd/_C.so`` (training, scoring, sampling)
+    and ``nanorlhf_amd/_serve.so`` (paged cache, attention over it, linear
+    attention, residual-stream kernels).  If an extension is missing on a
+    machine with a GPU this raises loudly — there is NO silent eager
     fallback on GPU.
   * CPU: a plain-PyTorch fp32 reference used by the CPU test suite and as
     the numerics oracle for the kernels.
@@ -12,45 +14,53 @@ from __future__ import annotations
 
 import importlib
 
-import torch  # noqa: F401  (must load before _C: provides libc10)
+import torch  # noqa: F401  (must load before the extensions: provides libc10)
 
-_EXT = None
-_EXT_ERR: Exception | None = None
-
-
-def _load():
-    global _EXT, _EXT_ERR
-    if _EXT is not None or _EXT_ERR is not None:
-        return _EXT
-    try:
-        _EXT = importlib.import_module("nanorlhf_amd._C")
-    except Exception as e:  # noqa: BLE001
-        _EXT_ERR = e
-        _EXT = None
-    return _EXT
+_LOADED: dict = {}
 
 
-def ext():
-    """The HIP extension module; raises loudly if unavailable."""
-    m = _load()
+def _load(name: str):
+    if name not in _LOADED:
+        try:
+            _LOADED[name] = (importlib.import_module(f"nanorlhf_amd.{name}"), None)
+        except Exception as e:  # noqa: BLE001
+            _LOADED[name] = (None, e)
+    return _LOADED[name]
+
+
+def _require(name: str):
+    m, err = _load(name)
     if m is None:
         raise RuntimeError(
-            "nanorlhf_amd._C HIP extension is not built/importable but a GPU op "
+            f"nanorlhf_amd.{name} HIP extension is not built/importable but a GPU op "
             "was requested. Build it in-tree with `python setup.py build_ext "
-            f"--inplace` (PYTORCH_ROCM_ARCH=gfx950). Original error: {_EXT_ERR!r}"
+            f"--inplace` (PYTORCH_ROCM_ARCH=gfx950). Original error: {err!r}"
         )
     return m
 
 
+def ext():
+    """The training/sampling extension; raises loudly if unavailable."""
+    return _require("_C")
+
+
+def serve_ext():
+    """The serving extension; raises loudly if unavailable."""
+    return _require("_serve")
+
+
 def ext_available() -> bool:
-    return _load() is not None
+    return all(_load(n)[0] is not None for n in ("_C", "_serve"))
 
 
-from .rmsnorm import add_rms_norm, rms_norm  # noqa: E402,F401
-from .rope import build_rope_cache, rope_apply  # noqa: E402,F401
-from .swiglu import swiglu  # noqa: E402,F401
+from .rmsnorm import (add_rms_norm, gated_norm, residual_group_norm,  # noqa: E402,F401
+                      rms_norm)
+from .rope import Rotation, build_rope_cache, rope_apply  # noqa: E402,F401
+from .swiglu import gelu_glu, swiglu  # noqa: E402,F401
 from .attention import flash_attn_varlen  # noqa: E402,F401
 from .logprob import token_logprob_entropy  # noqa: E402,F401
 from .adamw import FusedAdamW  # noqa: E402,F401
 from .sampling import sample_tokens  # noqa: E402,F401
-from .kvcache import kv_append, paged_attn_decode  # noqa: E402,F401
+from .kvcache import (kv_append, paged_attn, paged_attn_decode,  # noqa: E402,F401
+                      pad_head_dim, rotary_qkv)
+from .linear_attn import DecayTable, linear_attn_chunked, linear_attn_decode  # noqa: E402,F401

@@ -1,0 +1,105 @@
+"""Linear attention with a fixed decay per head and no denominator:
+
+    S_t = decay * S_(t-1) + k_t v_t^T        o_t = S_t^T q_t
+
+S [heads, dim, vdim] is 32-bit and lives in a state slot of its sequence.  q, k
+and v are columns of one projection row; SiLU (on all three), rotation (on q
+and k, 32-bit) and a factor on k are applied on the way in.
+
+GPU: csrc/linear_attn.hip.  Portions of prompts run in chunks of 64 tokens
+(chunk sums, a scan over chunks, chunk outputs); single tokens update their
+slot in place."""
+from __future__ import annotations
+
+import torch
+
+from . import serve_ext
+from .rope import rotate_pairs
+
+CHUNK = 64
+
+
+class DecayTable:
+    """Powers 0..CHUNK of each head's decay, [heads, CHUNK + 1] float32
+    (computed in 64-bit), one copy per device."""
+
+    def __init__(self, decay):
+        self.heads = len(decay)
+        d = torch.tensor(decay, dtype=torch.float64)[:, None]
+        n = torch.arange(CHUNK + 1, dtype=torch.float64)[None, :]
+        self._t = {"cpu": (d ** n).float()}
+
+    def on(self, device) -> torch.Tensor:
+        key = str(device)
+        if key not in self._t:
+            self._t[key] = self._t["cpu"].to(device)
+        return self._t[key]
+
+
+def _inputs(q, k, v, H, cs, interleaved, silu, kscale):
+    T = q.shape[0]
+    q, k, v = (t.reshape(T, H, -1).float() for t in (q, k, v))
+    if silu:
+        q, k, v = (torch.nn.functional.silu(t) for t in (q, k, v))
+    if cs is not None:
+        q = rotate_pairs(q, cs, interleaved)
+        k = rotate_pairs(k, cs, interleaved)
+    return q, k * kscale, v
+
+
+def linear_attn_chunked(q, k, v, decay: DecayTable, portions, state, *, cs=None,
+                        interleaved: bool = False, silu: bool = False,
+                        kscale: float = 1.0) -> torch.Tensor:
+    """q, k [T, H*D], v [T, H*V]: the tokens of `portions` (packed).  Each
+    portion goes on from its slot of state [slots, H, D, V] (from zero if it
+    starts its sequence) and leaves its last state there.  Returns [T, H*V]."""
+    o = torch.empty(v.shape, dtype=v.dtype, device=v.device)
+    if q.is_cuda:
+        serve_ext().linear_attn_chunked(q, k, v, decay.on(q.device), cs, interleaved, silu,
+                                        float(kscale), portions.chunks, portions.chunk_first,
+                                        portions.state_slots, portions.fresh, state, o)
+        return o
+    H, pw = decay.heads, decay.on("cpu")
+    q, k, v = _inputs(q, k, v, H, cs, interleaved, silu, kscale)
+    ch = portions.chunks
+    for b, slot in enumerate(portions.state_slots.tolist()):
+        S = state[slot] * 0 if portions.fresh[b] else state[slot].clone()
+        for c in range(int(portions.chunk_first[b]), int(portions.chunk_first[b + 1])):
+            r, n = int(ch[1, c]), int(ch[2, c])
+            qq, kk, vv = (t[r:r + n].transpose(0, 1) for t in (q, k, v))   # [H, n, .]
+            i = torch.arange(n)
+            gap = i[:, None] - i[None, :]
+            w = pw[:, gap.clamp(min=0)] * (gap >= 0)
+            inside = ((qq @ kk.transpose(1, 2)) * w) @ vv
+            ahead = (qq * pw[:, 1:n + 1, None]) @ S
+            o[r:r + n] = (inside + ahead).transpose(0, 1).reshape(n, -1).to(o.dtype)
+            S = pw[:, n, None, None] * S + (kk * pw[:, n - 1 - i, None]).transpose(1, 2) @ vv
+        state[slot] = S
+    return o
+
+
+def linear_attn_decode(q, k, v, decay: DecayTable, slots, seq_lens, state, *, cs=None,
+                       interleaved: bool = False, silu: bool = False, kscale: float = 1.0,
+                       gate=None, eps: float = 0.0, out=None) -> torch.Tensor:
+    """One token of each sequence (row b has slot slots[b]; seq_lens[b] == 1
+    starts from zero).  With `gate`, each head's output is divided by its root
+    mean square and multiplied by silu(gate).  Writes `out` (or a new tensor)."""
+    if out is None:
+        out = torch.empty(v.shape, dtype=v.dtype, device=v.device)
+    if q.is_cuda:
+        serve_ext().linear_attn_decode(q, k, v, decay.on(q.device), cs, interleaved, silu,
+                                       float(kscale), slots, seq_lens, state, gate,
+                                       float(eps), out)
+        return out
+    pw = decay.on("cpu")
+    q, k, v = _inputs(q, k, v, decay.heads, cs, interleaved, silu, kscale)
+    s = slots.long()
+    S = torch.where((seq_lens == 1)[:, None, None, None], 0.0, state[s])
+    S = pw[None, :, 1, None, None] * S + k[..., None] * v[..., None, :]
+    state[s] = S
+    o = (q[..., None] * S).sum(2)
+    if gate is not None:
+        o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)
+        o = o * torch.nn.functional.silu(gate.float()).view(o.shape)
+    out.copy_(o.reshape(o.shape[0], -1))
+    return out

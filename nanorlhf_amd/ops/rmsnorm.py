@@ -7,7 +7,7 @@ from __future__ import annotations
 
 import torch
 
-from . import ext
+from . import ext, serve_ext
 
 
 def _rms_norm_ref(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
@@ -67,3 +67,45 @@ def add_rms_norm(x: torch.Tensor, res: torch.Tensor | None, weight: torch.Tensor
         return _AddRMSNormFn.apply(x.contiguous(), res.contiguous(), weight, eps)
     h = x + res
     return rms_norm(h, weight, eps), h
+
+
+def _group_rms(x: torch.Tensor, groups: int, eps: float) -> torch.Tensor:
+    parts = x.float().unflatten(-1, (groups, x.shape[-1] // groups))
+    parts = parts * torch.rsqrt(parts.pow(2).mean(-1, keepdim=True) + eps)
+    return parts.flatten(-2)
+
+
+def residual_group_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, *,
+                        groups: int = 1, delta: torch.Tensor | None = None,
+                        mult: float = 1.0, embed: torch.Tensor | None = None,
+                        ids: torch.Tensor | None = None) -> torch.Tensor:
+    """Norm of a 32-bit residual stream, with the pending update fused in.
+
+    x [T, W] float32 is changed IN PLACE: set to embed[ids] if `ids` is given,
+    else x += mult * delta if `delta` is.  Returns, in the weight's dtype, x
+    split into `groups` equal parts, each divided by its own root mean square,
+    times weight [W]."""
+    if x.is_cuda:
+        return serve_ext().residual_group_norm(x, delta, embed, ids, weight, groups,
+                                               float(mult), float(eps))
+    if ids is not None:
+        x.copy_(embed[ids])
+    elif delta is not None:
+        x.add_(delta.float() * mult)
+    return (_group_rms(x, groups, eps) * weight.float()).to(weight.dtype)
+
+
+def gated_norm(x: torch.Tensor, weight: torch.Tensor | None, gate: torch.Tensor,
+               out: torch.Tensor, eps: float, *, groups: int = 1,
+               act: str = "silu") -> None:
+    """out[:] = grouped RMS norm of x (times weight) times act(gate); act is
+    "silu" or "sigmoid".  gate and out are column slices of wider rows."""
+    if x.is_cuda:
+        serve_ext().gated_norm(x, weight, gate, out, groups,
+                               {"silu": 0, "sigmoid": 1}[act], float(eps))
+        return
+    y = _group_rms(x, groups, eps)
+    if weight is not None:
+        y = y * weight.float()
+    g = gate.float()
+    out.copy_(y * (g * torch.sigmoid(g) if act == "silu" else torch.sigmoid(g)))

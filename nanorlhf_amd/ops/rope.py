@@ -9,7 +9,7 @@ from __future__ import annotations
 
 import torch
 
-from . import ext
+from . import ext, serve_ext
 
 
 def build_rope_cache(head_dim: int, max_pos: int, theta: float = 1e6,
@@ -57,3 +57,50 @@ def rope_apply(x: torch.Tensor, table: torch.Tensor, positions: torch.Tensor) ->
         # autograd-composable CPU path
         return _rope_ref(x, table, positions)
     return _rope_ref(x, table, positions)
+
+
+class Rotation:
+    """Rotary positions over the first `dims` dimensions, in either layout of
+    pairs: rotate-half (i with i + dims/2) or interleaved (2i with 2i + 1).
+
+    No table and no maximum position: the cos | sin rows of the tokens of one
+    forward are computed once (64-bit angle, 32-bit result) and shared by all
+    layers with the same base and dims."""
+
+    def __init__(self, dims: int, base: float, interleaved: bool = False):
+        if dims % 2:
+            raise ValueError(f"rotary dims must be even, got {dims}")
+        self.dims, self.base, self.interleaved = dims, float(base), interleaved
+        self.key = (dims, float(base))
+        i = torch.arange(dims // 2, dtype=torch.float64)
+        self._freqs = {"cpu": self.base ** (-2.0 * i / max(dims, 1))}
+
+    def freqs(self, device) -> torch.Tensor:
+        key = str(device)
+        if key not in self._freqs:
+            self._freqs[key] = self._freqs["cpu"].to(device)
+        return self._freqs[key]
+
+    def angles(self, positions: torch.Tensor) -> torch.Tensor:
+        """[T, dims] float32: cos of the dims/2 angles, then sin."""
+        f = self.freqs(positions.device)
+        if positions.is_cuda:
+            return serve_ext().rope_angles(positions, f)
+        a = positions.double().unsqueeze(1) * f
+        return torch.cat([a.cos(), a.sin()], dim=1).float()
+
+
+def rotate_pairs(x: torch.Tensor, cs: torch.Tensor, interleaved: bool,
+                 sign: float = 1.0) -> torch.Tensor:
+    """CPU reference: x [T, H, D] float32, cs [T, dims] with dims <= D."""
+    dims = cs.shape[1]
+    half = dims // 2
+    c = cs[:, None, :half]
+    s = cs[:, None, half:] * sign
+    if interleaved:
+        u, v = x[..., 0:dims:2], x[..., 1:dims:2]
+        rot = torch.stack([u * c - v * s, v * c + u * s], dim=-1).flatten(-2)
+    else:
+        u, v = x[..., :half], x[..., half:dims]
+        rot = torch.cat([u * c - v * s, v * c + u * s], dim=-1)
+    return torch.cat([rot, x[..., dims:]], dim=-1)

@@ -5,7 +5,7 @@ from __future__ import annotations
 
 import torch
 
-from . import ext
+from . import ext, serve_ext
 
 
 def _swiglu_ref(gate_up: torch.Tensor) -> torch.Tensor:
@@ -29,3 +29,17 @@ def swiglu(gate_up: torch.Tensor) -> torch.Tensor:
     if gate_up.is_cuda:
         return _SwigluFn.apply(gate_up.contiguous())
     return _swiglu_ref(gate_up)
+
+
+def gelu_glu(gate: torch.Tensor, up: torch.Tensor, out: torch.Tensor,
+             pad: int = 0, tail: int = 0) -> None:
+    """out[:, pad:pad+ff] = gelu_tanh(gate) * up; the pad columns ahead and the
+    tail columns behind are zeroed.  gate, up and out are column slices."""
+    if gate.is_cuda:
+        serve_ext().gelu_glu(gate, up, out, pad, tail)
+        return
+    ff = gate.shape[1]
+    out[:, :pad] = 0
+    out[:, pad + ff:] = 0
+    g = torch.nn.functional.gelu(gate.float(), approximate="tanh")
+    out[:, pad:pad + ff] = (g * up.float()).to(out.dtype)

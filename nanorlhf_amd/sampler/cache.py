@@ -1,37 +1,56 @@
-"""Paged KV-cache pool + page allocator.
+"""What the engine keeps of live sequences: KV pages and state slots.
 
-The vLLM-engine replacement's memory core.
-One (K, V) tensor pair per layer, [num_pages, page_size, Hkv, D] bf16,
-sized against 288 GB HBM3E.  Sequences own page lists; pages are recycled
-when a sequence finishes (continuous batching admits queued sequences into
-the freed space)."""
+Attention layers keep keys and values of every token in pages, one (K, V)
+tensor pair per layer, sized against 288 GB HBM3E; a sequence owns a list of
+pages.  Recurrent layers keep one 32-bit matrix per head in a slot; a sequence
+owns one slot number, valid in every such layer.  Pages and slot are recycled
+when a sequence finishes (continuous batching admits queued sequences into the
+freed space).  Neither is cleared: keys beyond a sequence's length are never
+visible, and a sequence's first token starts from a zero state."""
 from __future__ import annotations
 
+import numpy as np
 import torch
 
-from ..models.config import ModelConfig
+from ..models.config import KVSpec, StateSpec
 
 
 class PagedKVCache:
-    def __init__(self, cfg: ModelConfig, num_pages: int, page_size: int = 16,
-                 device="cpu", dtype=torch.bfloat16):
+    """layers[i] is (K, V) of an attention layer, [num_pages, page_size, heads,
+    k_dim] and d-major per page [num_pages, heads, v_dim, page_size] (so the
+    decode kernel's PV MFMA B-fragment is a contiguous 16-B load), or the state
+    of a recurrent layer, [num_slots, heads, dim, vdim] float32."""
+
+    def __init__(self, cfg, num_pages: int, page_size: int = 16, device="cpu",
+                 dtype=torch.bfloat16, num_slots: int = 0):
         self.page_size = page_size
         self.num_pages = num_pages
         self.device = device
-        kshape = (num_pages, page_size, cfg.num_kv_heads, cfg.head_dim)
-        # V is stored d-major within each page ([page][Hkv][D][page_size]) so
-        # the decode kernel's PV MFMA B-fragment is a contiguous 16-B load
-        vshape = (num_pages, cfg.num_kv_heads, cfg.head_dim, page_size)
-        self.layers = [
-            (torch.zeros(kshape, dtype=dtype, device=device),
-             torch.zeros(vshape, dtype=dtype, device=device))
-            for _ in range(cfg.num_layers)
-        ]
+        specs = cfg.cache_layers()
+        self.stateful = any(isinstance(s, StateSpec) for s in specs)
+        self.num_slots = num_slots if self.stateful else 0
+        if self.stateful and num_slots < 1:
+            raise ValueError("a model with recurrent layers needs state slots")
+        self.layers = [self._make(s, dtype) for s in specs]
         self._free = list(range(num_pages - 1, -1, -1))
+        self._free_slots = list(range(self.num_slots - 1, -1, -1))
+
+    def _make(self, s, dtype):
+        def zeros(*shape, dt=dtype):
+            return torch.zeros(shape, dtype=dt, device=self.device)
+
+        if isinstance(s, KVSpec):
+            return (zeros(self.num_pages, self.page_size, s.heads, s.k_dim),
+                    zeros(self.num_pages, s.heads, s.v_dim, self.page_size))
+        return zeros(self.num_slots, s.heads, s.dim, s.vdim, dt=torch.float32)
 
     @property
     def free_pages(self) -> int:
         return len(self._free)
+
+    @property
+    def free_slots(self) -> int:
+        return len(self._free_slots)
 
     def alloc(self, n: int) -> list[int]:
         if n > len(self._free):
@@ -41,23 +60,37 @@ class PagedKVCache:
     def free(self, pages: list[int]):
         self._free.extend(pages)
 
+    def release(self, seq: "SeqState"):
+        """Give back everything a sequence holds."""
+        self.free(seq.pages)
+        seq.pages = []
+        if seq.state_slot >= 0:
+            self._free_slots.append(seq.state_slot)
+            seq.state_slot = -1
+
     @staticmethod
-    def bytes_per_token(cfg: ModelConfig, dtype=torch.bfloat16) -> int:
+    def bytes_per_token(cfg, dtype=torch.bfloat16) -> int:
         esize = torch.tensor([], dtype=dtype).element_size()
-        return 2 * cfg.num_layers * cfg.num_kv_heads * cfg.head_dim * esize
+        return sum(s.heads * (s.k_dim + s.v_dim) * esize
+                   for s in cfg.cache_layers() if isinstance(s, KVSpec))
+
+    @staticmethod
+    def bytes_per_slot(cfg) -> int:
+        return sum(4 * s.heads * s.dim * s.vdim
+                   for s in cfg.cache_layers() if isinstance(s, StateSpec))
 
     @classmethod
-    def for_budget(cls, cfg: ModelConfig, max_tokens_total: int, page_size: int = 16,
-                   device="cpu", dtype=torch.bfloat16) -> "PagedKVCache":
+    def for_budget(cls, cfg, max_tokens_total: int, page_size: int = 16, device="cpu",
+                   dtype=torch.bfloat16, num_slots: int = 0) -> "PagedKVCache":
         pages = (max_tokens_total + page_size - 1) // page_size
-        return cls(cfg, pages, page_size, device, dtype)
+        return cls(cfg, pages, page_size, device, dtype, num_slots)
 
 
 class SeqState:
     """Book-keeping for one in-flight sequence."""
 
     __slots__ = ("uid", "tokens", "prompt_len", "pages", "finished", "out_index",
-                 "logprobs")
+                 "logprobs", "computed", "state_slot")
 
     def __init__(self, uid: int, prompt: list[int], out_index: int):
         self.uid = uid
@@ -67,6 +100,8 @@ class SeqState:
         self.finished = False
         self.out_index = out_index
         self.logprobs: list[float] = []  # per generated (response) token
+        self.computed = 0        # tokens whose KV and state the cache holds
+        self.state_slot = -1
 
     def __len__(self):
         return len(self.tokens)
@@ -78,7 +113,17 @@ class SeqState:
     def slot_of(self, pos: int, page_size: int) -> int:
         return self.pages[pos // page_size] * page_size + pos % page_size
 
+    def slots_for(self, start: int, end: int, page_size: int) -> np.ndarray:
+        pos = np.arange(start, end)
+        pages = np.asarray(self.pages, dtype=np.int64)
+        return pages[pos // page_size] * page_size + pos % page_size
+
     def ensure_capacity(self, pool: PagedKVCache, upto: int):
+        """Pages for `upto` tokens, and a state slot if the model keeps states."""
+        if pool.stateful and self.state_slot < 0:
+            if not pool._free_slots:
+                raise RuntimeError("no free state slot")
+            self.state_slot = pool._free_slots.pop()
         need = (upto + pool.page_size - 1) // pool.page_size
         if need > len(self.pages):
             self.pages.extend(pool.alloc(need - len(self.pages)))

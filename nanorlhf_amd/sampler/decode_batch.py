@@ -27,6 +27,7 @@ class DecodeBatch:
         self.seq_lens = torch.zeros(0, dtype=torch.int32, device=device)
         self.gen_count = torch.zeros(0, dtype=torch.int32, device=device)
         self.last_tok = torch.zeros(0, dtype=torch.long, device=device)
+        self.state_slots = torch.zeros(0, dtype=torch.int32, device=device)
         self.finished = torch.zeros(0, dtype=torch.bool, device=device)
         self.out = torch.zeros(0, max_tokens, dtype=torch.long, device=device)
         self.lp = torch.zeros(0, max_tokens, dtype=torch.float32, device=device)
@@ -70,6 +71,8 @@ class DecodeBatch:
         self.bt = torch.cat([self.bt, bt]) if len(self.seqs) else bt
         self.seq_lens = torch.cat([self.seq_lens, sl])
         self.last_tok = torch.cat([self.last_tok, lt])
+        self.state_slots = torch.cat([self.state_slots, torch.tensor(
+            [s.state_slot for s in seqs], dtype=torch.int32, device=self.device)])
         self.finished = torch.cat([self.finished, fin])
         self.out = torch.cat([self.out, out])
         self.lp = torch.cat([self.lp, lp])
@@ -130,8 +133,7 @@ class DecodeBatch:
             s.tokens = s.tokens[: s.prompt_len] + resp
             s.logprobs = lp_cpu[j, : len(resp)].tolist()
             s.finished = True
-            self.pool.free(s.pages)
-            s.pages = []
+            self.pool.release(s)
             retired.append(s)
         km = keep_mask.to(self.device)
         self.seqs = [s for r, s in enumerate(self.seqs) if not bool(fin[r])]
@@ -139,6 +141,7 @@ class DecodeBatch:
         self.seq_lens = self.seq_lens[km]
         self.gen_count = self.gen_count[km]
         self.last_tok = self.last_tok[km]
+        self.state_slots = self.state_slots[km]
         self.finished = self.finished[km]
         self.out = self.out[km]
         self.lp = self.lp[km]

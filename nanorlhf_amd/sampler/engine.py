@@ -16,10 +16,11 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
+import numpy as np
 import torch
 
 from .. import ops
-from ..models.qwen2 import AttnContext, CausalLM
+from ..models.qwen2 import AttnContext, Portions
 from ..models.lora import merge_for_rollout, unmerge
 from .cache import PagedKVCache, SeqState
 from .decode_batch import DecodeBatch
@@ -38,21 +39,32 @@ class SamplingParams:
 class SamplerEngine:
     KV_DTYPES = {"bf16": torch.bfloat16, "fp8_e4m3": torch.float8_e4m3fn}
 
-    def __init__(self, model: CausalLM, kv_pool_tokens: int, page_size: int = 16,
+    # device memory that state slots may take unless state_slots says otherwise
+    STATE_BYTES = 32 << 30
+
+    def __init__(self, model, kv_pool_tokens: int, page_size: int = 16,
                  max_num_seqs: int = 4096, prefill_chunk_tokens: int = 131072,
                  compact_interval: int = 32, use_graphs: bool = True,
                  kv_cache_dtype: str = "bf16",
-                 rollout_weight_dtype: str = "bf16"):
+                 rollout_weight_dtype: str = "bf16",
+                 state_slots: int | None = None):
+        if kv_cache_dtype not in model.kv_cache_dtypes:
+            raise ValueError(f"{type(model).__name__} caches {model.kv_cache_dtypes}, "
+                             f"not {kv_cache_dtype!r}")
         self.model = model
         self.device = next(model.parameters()).device
         self.dtype = next(model.parameters()).dtype
         kv_dtype = (self.KV_DTYPES[kv_cache_dtype]
                     if self.device.type == "cuda" or kv_cache_dtype != "bf16"
                     else self.dtype)
-        if self.device.type != "cuda" and kv_cache_dtype == "bf16":
-            kv_dtype = self.dtype  # CPU tests may run fp32 models
+        if kv_cache_dtype == "bf16":
+            kv_dtype = self.dtype  # float32 models cache float32
+        per_slot = PagedKVCache.bytes_per_slot(model.cfg)
+        if per_slot and state_slots is None:
+            state_slots = max(1, min(max_num_seqs, self.STATE_BYTES // per_slot))
         self.pool = PagedKVCache.for_budget(model.cfg, kv_pool_tokens, page_size,
-                                            device=self.device, dtype=kv_dtype)
+                                            device=self.device, dtype=kv_dtype,
+                                            num_slots=state_slots or 0)
         self.max_num_seqs = max_num_seqs
         self.prefill_chunk_tokens = prefill_chunk_tokens
         self.compact_interval = compact_interval
@@ -69,10 +81,6 @@ class SamplerEngine:
                                      if self.device.type == "cuda" else "bf16")
 
     # ----------------------------------------------------------------- utils
-    def _slots_for_range(self, seq: SeqState, start: int, end: int) -> list[int]:
-        ps = self.pool.page_size
-        return [seq.slot_of(p, ps) for p in range(start, end)]
-
     def _sample_from_hidden(self, hidden_last: torch.Tensor,
                             params: SamplingParams):
         """Returns (tokens [B], logprobs [B] fp32) — the chosen token's
@@ -95,14 +103,116 @@ class SamplerEngine:
         lp = logp.gather(1, tok.unsqueeze(1)).squeeze(1)
         return tok, lp
 
+    # ----------------------------------------------------------------- step
+    def _step_context(self, entries):
+        """Batch description of one step: single tokens first, then portions.
+        Returns (ids, ctx, first row of each entry)."""
+        ps = self.pool.page_size
+        order = sorted(range(len(entries)), key=lambda e: entries[e][1] != 1)
+        nd = sum(n == 1 for _, n in entries)
+        starts = [0] * len(entries)
+        ids, pos, slots, row = [], [], [], 0
+        for e in order:
+            s, n = entries[e]
+            a, b = s.computed, s.computed + n
+            if n < 1 or b > len(s.tokens):
+                raise ValueError(f"sequence {s.uid} has no tokens {a}..{b}")
+            s.ensure_capacity(self.pool, b)
+            starts[e] = row
+            row += n
+            ids.append(np.asarray(s.tokens[a:b], dtype=np.int64))
+            pos.append(np.arange(a, b))
+            slots.append(s.slots_for(a, b, ps))
+        seqs = [entries[e][0] for e in order]
+        lens = np.array([entries[e][1] for e in order])
+        P = max(len(s.pages) for s in seqs)
+        bt = np.zeros((len(seqs), P), dtype=np.int32)
+        for r, s in enumerate(seqs):
+            bt[r, :len(s.pages)] = s.pages
+        ints = {"bt": bt, "slot": np.array([s.state_slot for s in seqs]),
+                "len": np.array([s.computed for s in seqs]) + lens}
+        if nd < len(seqs):
+            plens = lens[nd:]
+            cu = np.concatenate([[0], np.cumsum(plens)])
+            per = -(-plens // ops.linear_attn.CHUNK)
+            owner = np.repeat(np.arange(len(plens)), per)
+            first = np.concatenate([[0], np.cumsum(per)])
+            off = (np.arange(len(owner)) - first[owner]) * ops.linear_attn.CHUNK
+            ints.update(cu=cu, row_seq=np.repeat(np.arange(len(plens)), plens),
+                        fresh=np.array([s.computed == 0 for s in seqs[nd:]]),
+                        chunks=np.stack([owner, cu[owner] + off,
+                                         np.minimum(plens[owner] - off,
+                                                    ops.linear_attn.CHUNK)]),
+                        first=first)
+        # one transfer for all int32 and one for all int64 arrays
+        dev32 = torch.from_numpy(np.concatenate(
+            [v.ravel() for v in ints.values()]).astype(np.int32)).to(self.device)
+        t, at = {}, 0
+        for k, v in ints.items():
+            t[k] = dev32[at:at + v.size].view(v.shape)
+            at += v.size
+        ids, pos, slots = torch.from_numpy(np.stack(
+            [np.concatenate(x) for x in (ids, pos, slots)])).to(self.device)
+        ctx = AttnContext(mode="step", positions=pos, slots=slots, kv_caches=self.pool.layers)
+        if nd:
+            ctx.block_tables, ctx.seq_lens = t["bt"][:nd], t["len"][:nd]
+            ctx.state_slots = t["slot"][:nd]
+        if nd < len(seqs):
+            ctx.portions = Portions(
+                cu=t["cu"], seq_lens=t["len"][nd:], block_tables=t["bt"][nd:],
+                row_seq=t["row_seq"], state_slots=t["slot"][nd:], fresh=t["fresh"],
+                chunks=t["chunks"], chunk_first=t["first"], max_q=int(lens[nd:].max()))
+        return ids, ctx, starts
+
+    @torch.no_grad()
+    def step(self, entries, on_layer=None):
+        """Run the next n tokens of each (sequence, n), all as one batch, from
+        what the cache holds of them; n == 1 is a decode step.
+
+        Returns (hidden [tokens, width], starts): entry e's rows are
+        starts[e] .. starts[e] + n - 1."""
+        ids, ctx, starts = self._step_context(entries)
+        ctx.on_layer = on_layer
+        hidden = self.model(ids, ctx)
+        for s, n in entries:
+            s.computed += n
+        return hidden, starts
+
     # -------------------------------------------------------------- prefill
     @torch.no_grad()
     def _prefill(self, seqs: list[SeqState], params: SamplingParams):
-        """Prefill `seqs` (packed varlen, chunked by token budget), append KV,
-        sample each sequence's first generated token."""
+        """Run the prompts of `seqs` within the token budget of a batch and
+        sample each one's first token.  Models with packed prefill run whole
+        prompts; the others are cut wherever the budget ends."""
+        if self.model.packed_prefill:
+            return self._prefill_packed(seqs, params)
+        todo = list(seqs)
+        while todo:
+            batch, room = [], self.prefill_chunk_tokens
+            for s in todo:
+                n = min(len(s) - s.computed, room)
+                if n:
+                    batch.append((s, n))
+                    room -= n
+            hidden, starts = self.step(batch)
+            done = [(s, r + n - 1) for (s, n), r in zip(batch, starts) if s.computed == len(s)]
+            if done:
+                rows = torch.tensor([r for _, r in done], device=self.device)
+                self._record_first([s for s, _ in done], hidden[rows], params)
+            todo = [s for s in todo if s.computed < s.prompt_len]
+
+    def _record_first(self, seqs, hidden, params):
+        tokens, lps = self._sample_from_hidden(hidden, params)
+        for s, t, l in zip(seqs, tokens.tolist(), lps.tolist()):
+            s.tokens.append(int(t))
+            s.logprobs.append(float(l))
+            if params.stop_token_id is not None and int(t) == params.stop_token_id:
+                s.finished = True
+
+    def _prefill_packed(self, seqs: list[SeqState], params: SamplingParams):
+        """Whole prompts as one packed varlen batch per token budget."""
         i = 0
         while i < len(seqs):
-            # pack a chunk of sequences up to the token budget
             chunk: list[SeqState] = []
             total = 0
             while i < len(seqs) and (not chunk or total + len(seqs[i]) <= self.prefill_chunk_tokens):
@@ -115,27 +225,22 @@ class SamplerEngine:
             cu = torch.zeros(len(chunk) + 1, dtype=torch.int32, device=self.device)
             cu[1:] = torch.cumsum(torch.tensor(lens, dtype=torch.int32, device=self.device), 0)
             pos = torch.cat([torch.arange(n, device=self.device) for n in lens])
-            slots = torch.tensor([sl for s in chunk for sl in self._slots_for_range(s, 0, len(s))],
-                                 dtype=torch.long, device=self.device)
+            slots = torch.from_numpy(np.concatenate(
+                [s.slots_for(0, len(s), self.pool.page_size) for s in chunk])).to(self.device)
             ctx = AttnContext(mode="prefill", positions=pos, cu_seqlens=cu,
                               max_seqlen=max(lens), kv_caches=self.pool.layers, slots=slots)
             hidden = self.model(ids, ctx)
-            last_idx = cu[1:].long() - 1
-            tokens, lps = self._sample_from_hidden(hidden[last_idx], params)
-            tok_list = tokens.tolist()
-            lp_list = lps.tolist()
-            for s, t, l in zip(chunk, tok_list, lp_list):
-                s.tokens.append(int(t))
-                s.logprobs.append(float(l))
-                if params.stop_token_id is not None and int(t) == params.stop_token_id:
-                    s.finished = True
+            for s in chunk:
+                s.computed = len(s)
+            self._record_first(chunk, hidden[cu[1:].long() - 1], params)
 
     # --------------------------------------------------------------- decode
     def _decode_step_eager(self, db: DecodeBatch, params: SamplingParams):
         ids, pos, slots, seq_lens, bt = db.step_inputs()
         ctx = AttnContext(mode="decode", positions=pos,
                           kv_caches=self.pool.layers, slots=slots,
-                          block_tables=bt, seq_lens=seq_lens)
+                          block_tables=bt, seq_lens=seq_lens,
+                          state_slots=db.state_slots)
         hidden = self.model(ids, ctx)
         tokens, lps = self._sample_from_hidden(hidden, params)
         db.commit(tokens, lps)
@@ -214,7 +319,8 @@ class SamplerEngine:
                             f"max_tokens {params.max_tokens}) but the KV pool "
                             f"has only {self.pool.num_pages}; raise "
                             "kv_pool_tokens or lower response_length")
-                    if need > self.pool.free_pages:
+                    if need > self.pool.free_pages or (
+                            self.pool.stateful and not self.pool.free_slots):
                         break
                     waiting.pop()
                     s.ensure_capacity(self.pool, len(s) + params.max_tokens)

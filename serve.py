@@ -5,7 +5,7 @@ update and thrown away); this exposes the same MI355X-native engine that
 drives training rollouts — paged fp8/bf16 KV, continuous batching,
 hipGraph-captured decode — behind a small HTTP API:
 
-    python serve.py --model /path/to/hf-qwen2-checkpoint [--port 8000]
+    python serve.py --model /path/to/checkpoint [--port 8000]
     python serve.py --preset qwen2.5-1.5b            # random-init (smoke)
 
 Endpoints:
@@ -29,19 +29,20 @@ import torch
 
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
-from nanorlhf_amd.models import CausalLM, get_config
+from nanorlhf_amd.models import build_model, get_config, load_model
 from nanorlhf_amd.sampler import SamplerEngine, SamplingParams
 
 
 class Server:
     def __init__(self, model, tokenizer, kv_pool_tokens: int,
-                 kv_cache_dtype: str = "fp8_e4m3"):
+                 kv_cache_dtype: str | None = None):
         self.model = model.eval()
         self.tokenizer = tokenizer
         dev = next(model.parameters()).device
         self.engine = SamplerEngine(
             model, kv_pool_tokens=kv_pool_tokens,
-            kv_cache_dtype=kv_cache_dtype if dev.type == "cuda" else "bf16")
+            kv_cache_dtype=(kv_cache_dtype or model.kv_cache_dtypes[0])
+            if dev.type == "cuda" else "bf16")
         self.lock = threading.Lock()   # one engine pass at a time
 
     def encode(self, prompt: str) -> list[int]:
@@ -108,17 +109,19 @@ def build_app(server: Server):
 
 
 def make_server(model_path: str | None, preset: str, kv_pool_tokens: int,
-                kv_cache_dtype: str = "fp8_e4m3") -> Server:
+                kv_cache_dtype: str | None = None) -> Server:
     tokenizer = None
     if model_path:
-        from nanorlhf_amd.data.tokenizer import load_tokenizer
-        from nanorlhf_amd.models.hf_import import load_pretrained
-        model = load_pretrained(model_path)
-        tokenizer = load_tokenizer(model_path)
+        model = load_model(model_path, **({} if torch.cuda.is_available()
+                                          else {"dtype": "float32"}))
+        if any(os.path.exists(os.path.join(model_path, f))
+               for f in ("tokenizer.json", "tokenizer_config.json")):
+            from nanorlhf_amd.data.tokenizer import load_tokenizer
+            tokenizer = load_tokenizer(model_path)
     else:
         cfg = get_config(preset, **({} if torch.cuda.is_available()
                                     else {"dtype": "float32"}))
-        model = CausalLM(cfg)
+        model = build_model(cfg)
     if torch.cuda.is_available():
         model = model.to("cuda").to(torch.bfloat16)
     return Server(model, tokenizer, kv_pool_tokens, kv_cache_dtype)
@@ -127,12 +130,14 @@ def make_server(model_path: str | None, preset: str, kv_pool_tokens: int,
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--model", type=str, default=None,
-                    help="local HF Qwen2 checkpoint dir (with tokenizer files)")
+                    help="checkpoint dir (config.json names the architecture; with "
+                         "no tokenizer files, prompts are bytes as ids)")
     ap.add_argument("--preset", type=str, default="qwen2.5-1.5b")
     ap.add_argument("--port", type=int, default=8000)
     ap.add_argument("--host", type=str, default="127.0.0.1")
     ap.add_argument("--kv-pool-tokens", type=int, default=2_000_000)
-    ap.add_argument("--kv-dtype", type=str, default="fp8_e4m3")
+    ap.add_argument("--kv-dtype", type=str, default=None,
+                    help="fp8_e4m3 | bf16 (default: the model's first choice)")
     args = ap.parse_args()
     import uvicorn
     server = make_server(args.model, args.preset, args.kv_pool_tokens,
