@@ -12,6 +12,8 @@ sampler) -> reward model pass -> scoring pass (policy+ref logprobs, fused
 HIP logprob kernel) -> PPO minibatch update (HIP AdamW).
 
 Usage:  python bench.py [--gpus N] [--steps K] [--warmup W]
+        python bench.py --serving [SIZE,...]    prefill and decode throughput of
+            Gonurax beside Qwen2 at equal size, one JSON line per measurement
 Multi-GPU: launched by the driver via torch.distributed.run, one rank per
 GPU over RCCL; rank 0 prints ONE JSON line.
 """
@@ -52,7 +54,15 @@ def main():
     ap.add_argument("--rollout-weight-dtype", type=str, default="bf16",
                     help="bf16 (default) | fp8_e4m3 (e4m3 merged rollout "
                          "weights; secondary measurement until promoted)")
+    ap.add_argument("--serving", nargs="?", const="all", default=None, metavar="SIZE,...",
+                    help="measure serving instead: prefill and decode tokens/s of Gonurax "
+                         "and of Qwen2 at equal size (random weights)")
+    ap.add_argument("--serving-models", default="gonurax,qwen2")
     args = ap.parse_args()
+    if args.serving:
+        from nanorlhf_amd.utils.serving_bench import run
+        return run(args.serving, args.serving_models.split(","), max(args.steps, 1),
+                   max(args.warmup, 1))
 
     from nanorlhf_amd.algos import grpo
     from nanorlhf_amd.algos.grpo import GRPOConfig

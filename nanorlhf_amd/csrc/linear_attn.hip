@@ -9,7 +9,11 @@
 //                   sequence's slot (or zero) and back into it;
 //   3. chunk_out:   decayed (q k^T) v inside a chunk plus q times the state
 //                   ahead of it, in parallel.
-// Products run on the matrix cores: float32 MFMA here, exact to 32-bit.
+// Products run on the matrix cores.  float32 inputs use float32 MFMA.  bf16
+// inputs use bf16 MFMA on split operands: whatever is 32-bit (rotated and
+// decayed q and k, decayed scores, the state) is the sum of two bf16 numbers,
+// hi + lo, and a product is the sum of the significant cross terms, so about
+// 16 bits of every operand count; v is bf16 as the projection left it.
 //
 // Single tokens (decode) update the state in place: one workgroup per
 // (sequence, head) streams S once through registers.
@@ -151,7 +155,7 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
 template <typename T, int DP>
 __global__ __launch_bounds__(256) void chunk_out_kernel(
     const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v, Source s,
-    Chunks ch, const float* __restrict__ pw, const float* __restrict__ ws, T* __restrict__ o) {
+    Chunks ch, const float* __restrict__ pw, const float* __restrict__ ws, T* __restrict__ o, long ldo) {
   constexpr int KS = DP + 4, VS = VBLK + 16, PS = CHUNK + 4;
   __shared__ float kt[CHUNK * KS], vt[CHUNK * VS], pt[4][16 * PS], pws[CHUNK + 1];
   const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VBLK;
@@ -224,8 +228,400 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
 #pragma unroll
     for (int r = 0; r < 4; r++) {
       const int i = 16 * w + 4 * hi + r, e = v0 + 16 * t + lo;
-      if (i < n && e < s.V) stf(o + (t0 + i) * (long)s.H * s.V + h * s.V + e, acc[t][r]);
+      if (i < n && e < s.V) stf(o + (t0 + i) * ldo + h * s.V + e, acc[t][r]);
     }
+}
+
+// ===================================================== bf16: split operands
+typedef __bf16 bf16x8l __attribute__((ext_vector_type(8)));
+typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+
+DEVINL f32x4 mfma16l(bf16x8l a, bf16x8l b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+DEVINL bf16x8l frag(const short* p) { return *reinterpret_cast<const bf16x8l*>(p); }
+DEVINL float silu_fast(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+
+// x = hi + lo, both bf16
+DEVINL void split4(const float* x, s16x4& hi, s16x4& lo) {
+#pragma unroll
+  for (int j = 0; j < 4; j++) {
+    hi[j] = f2bf(x[j]);
+    lo[j] = f2bf(x[j] - bf2f(hi[j]));
+  }
+}
+
+// Eight elements of one q or k row, as two runs of four: a at element ea, b at
+// eb.  Run g holds whole rotation pairs (with `vec`; without it, elements 8g..
+// 8g+7 one by one).  Elements past D are 0.
+DEVINL void load_runs(const short* row, int g, const Source& s, const float* cs, bool vec,
+                      float* a, float* b, int& ea, int& eb) {
+  if (!vec) {
+    ea = 8 * g;
+    eb = ea + 4;
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      a[j] = ea + j < s.D ? load_qk(row, ea + j, s, cs) : 0.f;
+      b[j] = eb + j < s.D ? load_qk(row, eb + j, s, cs) : 0.f;
+    }
+    return;
+  }
+  const int half = s.rdims >> 1, p = 4 * g;      // first of four pairs
+  const bool rot = p < half;
+  if (s.interleaved || !rot) {
+    ea = rot || s.interleaved ? 2 * p : s.rdims + 2 * (p - half);
+    eb = ea + 4;
+  } else {
+    ea = p;
+    eb = half + p;
+  }
+#pragma unroll
+  for (int j = 0; j < 4; j++) a[j] = b[j] = 0.f;
+  if (ea < s.D) ldv<4>(row + ea, a);
+  if (eb < s.D) ldv<4>(row + eb, b);
+  if (s.silu) {
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      a[j] = silu_fast(a[j]);
+      b[j] = silu_fast(b[j]);
+    }
+  }
+  if (!rot) return;
+  float c[4], sn[4];
+  ldv<4>(cs + p, c);
+  ldv<4>(cs + half + p, sn);
+  if (s.interleaved) {
+#pragma unroll
+    for (int j = 0; j < 4; j += 2) {
+      const float u = a[j], v = a[j + 1];
+      a[j] = u * c[j / 2] - v * sn[j / 2];
+      a[j + 1] = v * c[j / 2] + u * sn[j / 2];
+      const float x = b[j], y = b[j + 1];
+      b[j] = x * c[2 + j / 2] - y * sn[2 + j / 2];
+      b[j + 1] = y * c[2 + j / 2] + x * sn[2 + j / 2];
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      const float u = a[j], v = b[j];
+      a[j] = u * c[j] - v * sn[j];
+      b[j] = v * c[j] + u * sn[j];
+    }
+  }
+}
+
+constexpr int TS = CHUNK + 8;    // LDS row of a [feature][token] tile
+
+// vt[e][j] = v_j[v0 + e], 0 past the chunk's tokens and past V
+template <int VB, int NT>
+DEVINL void stage_v(short* vt, const short* v, const Source& s, long t0, int n, int h, int v0,
+                    bool vec) {
+  for (int i = threadIdx.x; i < (CHUNK / 4) * (VB / 4); i += NT) {
+    const int e = (i % (VB / 4)) * 4, j = (i / (VB / 4)) * 4;
+    float x[4][4];
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      const short* row = v + (t0 + j + r) * s.ld + h * s.V + v0 + e;
+#pragma unroll
+      for (int c = 0; c < 4; c++) x[r][c] = 0.f;
+      if (j + r < n) {
+        if (vec) {
+          if (v0 + e < s.V) ldv<4>(row, x[r]);
+        } else {
+#pragma unroll
+          for (int c = 0; c < 4; c++)
+            if (v0 + e + c < s.V) x[r][c] = ldf(row + c);
+        }
+      }
+      if (s.silu) {
+#pragma unroll
+        for (int c = 0; c < 4; c++) x[r][c] = silu_fast(x[r][c]);
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < 4; c++) {
+      const float col[4] = {x[0][c], x[1][c], x[2][c], x[3][c]};
+      stv<4>(vt + (e + c) * TS + j, col);
+    }
+  }
+}
+
+// ws [chunks, H, V, DP]: what a chunk adds, feature-major
+template <int DP, int VB>
+__global__ __launch_bounds__(256) void chunk_state_split_kernel(
+    const short* __restrict__ k, const short* __restrict__ v, Source s, Chunks ch,
+    const float* __restrict__ pw, float* __restrict__ ws, bool vec) {
+  __shared__ __attribute__((aligned(16))) short kt[2][DP * TS], vt[VB * TS];
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
+  const int n = ch.len[c];
+  const long t0 = ch.row[c];
+  const float* pwh = pw + h * (CHUNK + 1);
+  stage_v<VB, 256>(vt, v, s, t0, n, h, v0, vec);
+  for (int i = threadIdx.x; i < (CHUNK / 4) * (DP / 8); i += 256) {
+    const int g = i % (DP / 8), j = (i / (DP / 8)) * 4;
+    float a[4][4], b[4][4];
+    int ea = 8 * g, eb = ea + 4;
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      const bool live = j + r < n;
+      const long t = t0 + (live ? j + r : 0);
+      load_runs(k + t * s.ld + h * s.D, g, s, s.cs + t * s.rdims, vec, a[r], b[r], ea, eb);
+      const float m = live ? s.kscale * pwh[n - 1 - j - r] : 0.f;
+#pragma unroll
+      for (int q = 0; q < 4; q++) {
+        a[r][q] *= m;
+        b[r][q] *= m;
+      }
+    }
+#pragma unroll
+    for (int q = 0; q < 4; q++) {
+      const float x[4] = {a[0][q], a[1][q], a[2][q], a[3][q]};
+      const float y[4] = {b[0][q], b[1][q], b[2][q], b[3][q]};
+      s16x4 hi, lo;
+      split4(x, hi, lo);
+      *reinterpret_cast<s16x4*>(&kt[0][(ea + q) * TS + j]) = hi;
+      *reinterpret_cast<s16x4*>(&kt[1][(ea + q) * TS + j]) = lo;
+      split4(y, hi, lo);
+      *reinterpret_cast<s16x4*>(&kt[0][(eb + q) * TS + j]) = hi;
+      *reinterpret_cast<s16x4*>(&kt[1][(eb + q) * TS + j]) = lo;
+    }
+  }
+  __syncthreads();
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int lo = lane & 15, hi = lane >> 4;
+  constexpr int CW = VB / 64;                  // v tiles per wave
+  bf16x8l vf[CW][2];
+#pragma unroll
+  for (int q = 0; q < CW; q++)
+#pragma unroll
+    for (int ks = 0; ks < 2; ks++)
+      vf[q][ks] = frag(&vt[((w * CW + q) * 16 + lo) * TS + 32 * ks + 8 * hi]);
+  float* u = ws + ((long)c * s.H + h) * s.V * DP;
+#pragma unroll 2
+  for (int rt = 0; rt < DP / 16; rt++) {
+    bf16x8l kf[2][2];
+#pragma unroll
+    for (int pl = 0; pl < 2; pl++)
+#pragma unroll
+      for (int ks = 0; ks < 2; ks++)
+        kf[pl][ks] = frag(&kt[pl][(16 * rt + lo) * TS + 32 * ks + 8 * hi]);
+#pragma unroll
+    for (int q = 0; q < CW; q++) {
+      f32x4 acc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < 2; ks++) {
+        acc = mfma16l(kf[1][ks], vf[q][ks], acc);
+        acc = mfma16l(kf[0][ks], vf[q][ks], acc);
+      }
+      const int e = v0 + (w * CW + q) * 16 + lo;
+      if (e < s.V) *reinterpret_cast<f32x4*>(u + (long)e * DP + 16 * rt + 4 * hi) = acc;
+    }
+  }
+}
+
+// in place: what a chunk adds -> the state ahead of it, as hi | lo << 16.
+// The slot itself is exchanged in full float32, [D][V].
+__global__ __launch_bounds__(256) void chunk_scan_split_kernel(
+    float* __restrict__ ws, float* __restrict__ state, Chunks ch,
+    const int* __restrict__ slots, const int* __restrict__ fresh,
+    const float* __restrict__ pw, int H, int D, int V, int DP) {
+  constexpr int AHEAD = 8;
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int e = blockIdx.z * 256 + threadIdx.x;
+  if (e >= V * DP) return;
+  const int vi = e / DP, d = e % DP;
+  const bool real = d < D;
+  float* st = state + (((long)slots[b] * H + h) * D + (real ? d : 0)) * V + vi;
+  const float* pwh = pw + h * (CHUNK + 1);
+  float s = (fresh[b] || !real) ? 0.f : *st;
+  const int c0 = ch.first[b], c1 = ch.first[b + 1];
+  const long step = (long)H * V * DP;
+  float* p = ws + ((long)c0 * H + h) * V * DP + e;
+  for (int c = c0; c < c1; c += AHEAD) {
+    float u[AHEAD];
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) u[i] = c + i < c1 ? p[i * step] : 0.f;
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) {
+      if (c + i >= c1) break;
+      const short hi = f2bf(s), lo = f2bf(s - bf2f(hi));
+      reinterpret_cast<unsigned*>(p)[i * step] =
+          (unsigned)(unsigned short)hi | ((unsigned)(unsigned short)lo << 16);
+      s = pwh[ch.len[c + i]] * s + u[i];
+    }
+    p += AHEAD * step;
+  }
+  if (real) *st = s;
+}
+
+// One workgroup: one chunk, one head, VB columns of v.  Everything is computed
+// transposed (a lane holds one token's consecutive columns).  With a gate (V
+// <= VB), the head's output leaves normed and gated.
+template <int DP, int VB>
+__global__ __launch_bounds__(512) void chunk_out_split_kernel(
+    const short* __restrict__ q, const short* __restrict__ k, const short* __restrict__ v,
+    Source s, Chunks ch, const float* __restrict__ pw, const unsigned* __restrict__ ws,
+    const short* __restrict__ gate, long ldg, float eps, short* __restrict__ o, long ldo,
+    bool vec) {
+  constexpr int QS = DP + 8;
+  constexpr int KR = 2 * CHUNK * (QS > TS ? QS : TS);
+  constexpr int CT = VB / 16;             // v tiles: 4 or 8
+  constexpr int RW = CT / 2;              // token tiles per wave
+  __shared__ __attribute__((aligned(16))) short qt[2][CHUNK * QS], kreg[KR], vt[VB * TS];
+  __shared__ float pws[CHUNK + 1], red[CT][CHUNK];
+  short* kt[2] = {kreg, kreg + CHUNK * QS};
+  short* pt[2] = {kreg, kreg + CHUNK * TS};    // scores take the keys' place
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
+  const int n = ch.len[c];
+  const long t0 = ch.row[c];
+  if (threadIdx.x <= CHUNK) pws[threadIdx.x] = pw[h * (CHUNK + 1) + threadIdx.x];
+  for (int i = threadIdx.x; i < CHUNK * (DP / 8); i += 512) {
+    const int g = i % (DP / 8), j = i / (DP / 8);
+    const long t = t0 + (j < n ? j : 0);
+    float a[4], b[4];
+    int ea, eb;
+    s16x4 hi, lo;
+    load_runs(q + t * s.ld + h * s.D, g, s, s.cs + t * s.rdims, vec, a, b, ea, eb);
+    split4(a, hi, lo);
+    *reinterpret_cast<s16x4*>(&qt[0][j * QS + ea]) = hi;
+    *reinterpret_cast<s16x4*>(&qt[1][j * QS + ea]) = lo;
+    split4(b, hi, lo);
+    *reinterpret_cast<s16x4*>(&qt[0][j * QS + eb]) = hi;
+    *reinterpret_cast<s16x4*>(&qt[1][j * QS + eb]) = lo;
+    load_runs(k + t * s.ld + h * s.D, g, s, s.cs + t * s.rdims, vec, a, b, ea, eb);
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+      a[r] *= s.kscale;
+      b[r] *= s.kscale;
+    }
+    split4(a, hi, lo);
+    *reinterpret_cast<s16x4*>(&kt[0][j * QS + ea]) = hi;
+    *reinterpret_cast<s16x4*>(&kt[1][j * QS + ea]) = lo;
+    split4(b, hi, lo);
+    *reinterpret_cast<s16x4*>(&kt[0][j * QS + eb]) = hi;
+    *reinterpret_cast<s16x4*>(&kt[1][j * QS + eb]) = lo;
+  }
+  stage_v<VB, 512>(vt, v, s, t0, n, h, v0, vec);
+  __syncthreads();
+
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int lo = lane & 15, hi = lane >> 4;
+  const int ct = w % CT, r0 = (w / CT) * RW;
+  const int e0 = v0 + 16 * ct;
+  f32x4 acc[RW];
+#pragma unroll
+  for (int r = 0; r < RW; r++) acc[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+  // state ahead of the chunk, times q
+  const unsigned* sp = ws + (((long)c * s.H + h) * s.V + min(e0 + lo, s.V - 1)) * DP;
+#pragma unroll 4
+  for (int ks = 0; ks < DP / 32; ks++) {
+    u32x4 x = *reinterpret_cast<const u32x4*>(sp + 32 * ks + 8 * hi);
+    u32x4 y = *reinterpret_cast<const u32x4*>(sp + 32 * ks + 8 * hi + 4);
+    if (e0 + lo >= s.V) x = y = u32x4{0u, 0u, 0u, 0u};
+    union { unsigned u[4]; bf16x8l f; } sh, sl;
+    sh.u[0] = __builtin_amdgcn_perm(x[1], x[0], 0x05040100);
+    sh.u[1] = __builtin_amdgcn_perm(x[3], x[2], 0x05040100);
+    sh.u[2] = __builtin_amdgcn_perm(y[1], y[0], 0x05040100);
+    sh.u[3] = __builtin_amdgcn_perm(y[3], y[2], 0x05040100);
+    sl.u[0] = __builtin_amdgcn_perm(x[1], x[0], 0x07060302);
+    sl.u[1] = __builtin_amdgcn_perm(x[3], x[2], 0x07060302);
+    sl.u[2] = __builtin_amdgcn_perm(y[1], y[0], 0x07060302);
+    sl.u[3] = __builtin_amdgcn_perm(y[3], y[2], 0x07060302);
+#pragma unroll
+    for (int r = 0; r < RW; r++) {
+      const int at = (16 * (r0 + r) + lo) * QS + 32 * ks + 8 * hi;
+      const bf16x8l qh = frag(&qt[0][at]), ql = frag(&qt[1][at]);
+      acc[r] = mfma16l(sl.f, qh, acc[r]);
+      acc[r] = mfma16l(sh.f, ql, acc[r]);
+      acc[r] = mfma16l(sh.f, qh, acc[r]);
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RW; r++) acc[r] *= pws[16 * (r0 + r) + lo + 1];
+  // scores of this wave's two tiles (token tile it, key tiles jt, jt + 1)
+  const int it = w >> 1, jt = (w & 1) * 2;
+  f32x4 sc[2];
+#pragma unroll
+  for (int x = 0; x < 2; x++) {
+    sc[x] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (jt + x > it) continue;
+#pragma unroll 4
+    for (int ks = 0; ks < DP / 32; ks++) {
+      const int qa = (16 * it + lo) * QS + 32 * ks + 8 * hi;
+      const int ka = (16 * (jt + x) + lo) * QS + 32 * ks + 8 * hi;
+      const bf16x8l qh = frag(&qt[0][qa]), ql = frag(&qt[1][qa]);
+      const bf16x8l kh = frag(&kt[0][ka]), kl = frag(&kt[1][ka]);
+      sc[x] = mfma16l(kl, qh, sc[x]);
+      sc[x] = mfma16l(kh, ql, sc[x]);
+      sc[x] = mfma16l(kh, qh, sc[x]);
+    }
+  }
+  __syncthreads();                 // every wave is done with the keys
+#pragma unroll
+  for (int x = 0; x < 2; x++) {
+    const int i = 16 * it + lo, j = 16 * (jt + x) + 4 * hi;
+    float p[4];
+#pragma unroll
+    for (int r = 0; r < 4; r++) p[r] = i >= j + r ? sc[x][r] * pws[max(i - j - r, 0)] : 0.f;
+    s16x4 ph, pl;
+    split4(p, ph, pl);
+    *reinterpret_cast<s16x4*>(&pt[0][i * TS + j]) = ph;
+    *reinterpret_cast<s16x4*>(&pt[1][i * TS + j]) = pl;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int r = 0; r < RW; r++)
+    for (int ks = 0; ks <= (r0 + r) / 2; ks++) {
+      const bf16x8l vf = frag(&vt[(16 * ct + lo) * TS + 32 * ks + 8 * hi]);
+      const int at = (16 * (r0 + r) + lo) * TS + 32 * ks + 8 * hi;
+      acc[r] = mfma16l(vf, frag(&pt[1][at]), acc[r]);
+      acc[r] = mfma16l(vf, frag(&pt[0][at]), acc[r]);
+    }
+  float inv[RW];
+  if (gate) {
+#pragma unroll
+    for (int r = 0; r < RW; r++) {
+      float ss = acc[r][0] * acc[r][0] + acc[r][1] * acc[r][1] + acc[r][2] * acc[r][2] +
+                 acc[r][3] * acc[r][3];
+      ss += __shfl_xor(ss, 16);
+      ss += __shfl_xor(ss, 32);
+      if (hi == 0) red[ct][16 * (r0 + r) + lo] = ss;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < RW; r++) {
+      float ss = 0.f;
+#pragma unroll
+      for (int x = 0; x < CT; x++) ss += red[x][16 * (r0 + r) + lo];
+      inv[r] = 1.f / sqrtf(ss / (float)s.V + eps);
+    }
+  }
+  const int e = e0 + 4 * hi;
+#pragma unroll
+  for (int r = 0; r < RW; r++) {
+    const int i = 16 * (r0 + r) + lo;
+    if (i >= n || e >= s.V) continue;
+    float x[4];
+#pragma unroll
+    for (int j = 0; j < 4; j++) x[j] = acc[r][j];
+    short* dst = o + (t0 + i) * ldo + h * s.V + e;
+    if (vec) {
+      if (gate) {
+        float g[4];
+        ldv<4>(gate + (t0 + i) * ldg + h * s.V + e, g);
+#pragma unroll
+        for (int j = 0; j < 4; j++) x[j] *= inv[r] * silu_fast(g[j]);
+      }
+      stv<4>(dst, x);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        if (e + j >= s.V) continue;
+        if (gate) x[j] *= inv[r] * silu_fast(ldf(gate + (t0 + i) * ldg + h * s.V + e + j));
+        stf(dst + j, x[j]);
+      }
+    }
+  }
 }
 
 // ------------------------------------------------------------- one token
@@ -334,13 +730,15 @@ static void check_ints(const torch::Tensor& t, long n) {
   TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt && t.is_contiguous() && t.numel() == n);
 }
 
-// o [T, H * V] <- portions described by chunks (int32 [3, n]: sequence, first
-// row, length), first (int32 [B + 1]), slots and fresh (int32 [B])
+// o [T, H * V] (any row stride) <- portions described by chunks (int32 [3, n]:
+// sequence, first row, length), first (int32 [B + 1]), slots and fresh (int32
+// [B]).  With a gate, each head's output is divided by its root mean square and
+// multiplied by silu(gate): bf16 and V <= 128 only.
 void linear_attn_chunked(torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor pw,
                          c10::optional<torch::Tensor> cs, bool interleaved, bool silu,
                          double kscale, torch::Tensor chunks, torch::Tensor first,
                          torch::Tensor slots, torch::Tensor fresh, torch::Tensor state,
-                         torch::Tensor o) {
+                         c10::optional<torch::Tensor> gate, double eps, torch::Tensor o) {
   const Source s = make_source(q, k, v, pw, cs, interleaved, silu, kscale);
   check_state(state, s);
   const long n = chunks.size(1), B = slots.numel();
@@ -348,10 +746,15 @@ void linear_attn_chunked(torch::Tensor q, torch::Tensor k, torch::Tensor v, torc
   check_ints(first, B + 1);
   check_ints(slots, B);
   check_ints(fresh, B);
-  TORCH_CHECK(o.is_contiguous() && o.scalar_type() == q.scalar_type() && o.size(0) == q.size(0) &&
+  TORCH_CHECK(o.stride(1) == 1 && o.scalar_type() == q.scalar_type() && o.size(0) == q.size(0) &&
               o.size(1) == (long)s.H * s.V);
+  if (gate.has_value())
+    TORCH_CHECK(q.scalar_type() == torch::kBFloat16 && s.V <= 128 && gate->stride(1) == 1 &&
+                gate->scalar_type() == q.scalar_type() && gate->sizes() == o.sizes());
   if (n == 0) return;
-  auto ws = torch::empty({n, s.H, s.D, s.V}, state.options());
+  const int DP = s.D <= 32 ? 32 : s.D <= 64 ? 64 : s.D <= 128 ? 128 : 256;
+  const bool split = q.scalar_type() == torch::kBFloat16;
+  auto ws = torch::empty({n, s.H, s.V, split ? DP : s.D}, state.options());
   int* cp = chunks.data_ptr<int>();
   const Chunks ch{cp, cp + n, cp + 2 * n, first.data_ptr<int>()};
   auto stream = at::hip::getCurrentHIPStream();
@@ -359,30 +762,55 @@ void linear_attn_chunked(torch::Tensor q, torch::Tensor k, torch::Tensor v, torc
   const int DV = s.D * s.V;
   const float* pwp = pw.data_ptr<float>();
   float* wsp = ws.data_ptr<float>();
-#define PHASES(TT, DP)                                                                         \
+  if (split) {
+    auto al = [](const void* p) { return ((uintptr_t)p % 8) == 0; };
+    const bool vec = s.D % 4 == 0 && s.V % 4 == 0 && s.rdims % 8 == 0 && s.ld % 4 == 0 &&
+                     o.stride(0) % 4 == 0 && al(q.data_ptr()) && al(k.data_ptr()) &&
+                     al(v.data_ptr()) && al(o.data_ptr()) && ((uintptr_t)s.cs % 16) == 0 &&
+                     (!gate.has_value() || (gate->stride(0) % 4 == 0 && al(gate->data_ptr())));
+    const short* gp = gate.has_value() ? (const short*)gate->data_ptr() : nullptr;
+    const long ldg = gate.has_value() ? gate->stride(0) : 0;
+#define SPLIT(DD, VB)                                                                           \
+  do {                                                                                          \
+    const dim3 sg(n, s.H, (s.V + VB - 1) / VB);                                                 \
+    hipLaunchKernelGGL((chunk_state_split_kernel<DD, VB>), sg, dim3(256), 0, stream,            \
+                       (const short*)k.data_ptr(), (const short*)v.data_ptr(), s, ch, pwp, wsp, \
+                       vec);                                                                    \
+    hipLaunchKernelGGL(chunk_scan_split_kernel, dim3(B, s.H, (s.V * DD + 255) / 256),           \
+                       dim3(256), 0, stream, wsp, state.data_ptr<float>(), ch,                  \
+                       slots.data_ptr<int>(), fresh.data_ptr<int>(), pwp, s.H, s.D, s.V, DD);   \
+    hipLaunchKernelGGL((chunk_out_split_kernel<DD, VB>), sg, dim3(512), 0, stream,              \
+                       (const short*)q.data_ptr(), (const short*)k.data_ptr(),                  \
+                       (const short*)v.data_ptr(), s, ch, pwp, (const unsigned*)wsp, gp, ldg,   \
+                       (float)eps, (short*)o.data_ptr(), (long)o.stride(0), vec);               \
+  } while (0)
+#define SPLIT_V(DD) do { if (s.V <= 64) SPLIT(DD, 64); else SPLIT(DD, 128); } while (0)
+    if (DP == 32) SPLIT_V(32);
+    else if (DP == 64) SPLIT_V(64);
+    else if (DP == 128) SPLIT_V(128);
+    else SPLIT_V(256);
+#undef SPLIT_V
+#undef SPLIT
+    HIP_CHECK_LAST();
+    return;
+  }
+  TORCH_CHECK(q.scalar_type() == torch::kFloat32);
+#define PHASES(DD)                                                                             \
   do {                                                                                         \
-    hipLaunchKernelGGL((chunk_state_kernel<TT, DP>), grid, dim3(256), 0, stream,               \
-                       (const TT*)k.data_ptr(), (const TT*)v.data_ptr(), s, ch, pwp, wsp);     \
+    hipLaunchKernelGGL((chunk_state_kernel<float, DD>), grid, dim3(256), 0, stream,            \
+                       (const float*)k.data_ptr(), (const float*)v.data_ptr(), s, ch, pwp, wsp); \
     hipLaunchKernelGGL(chunk_scan_kernel, dim3(B, s.H, (DV + 255) / 256), dim3(256), 0, stream, \
                        wsp, state.data_ptr<float>(), ch, slots.data_ptr<int>(),                \
                        fresh.data_ptr<int>(), pwp, s.H, DV);                                   \
-    hipLaunchKernelGGL((chunk_out_kernel<TT, DP>), grid, dim3(256), 0, stream,                 \
-                       (const TT*)q.data_ptr(), (const TT*)k.data_ptr(),                       \
-                       (const TT*)v.data_ptr(), s, ch, pwp, wsp, (TT*)o.data_ptr());           \
+    hipLaunchKernelGGL((chunk_out_kernel<float, DD>), grid, dim3(256), 0, stream,              \
+                       (const float*)q.data_ptr(), (const float*)k.data_ptr(),                 \
+                       (const float*)v.data_ptr(), s, ch, pwp, wsp, (float*)o.data_ptr(),      \
+                       (long)o.stride(0));                                                     \
   } while (0)
-#define BY_D(TT)                            \
-  do {                                      \
-    if (s.D <= 32) PHASES(TT, 32);          \
-    else if (s.D <= 64) PHASES(TT, 64);     \
-    else if (s.D <= 128) PHASES(TT, 128);   \
-    else PHASES(TT, 256);                   \
-  } while (0)
-  if (q.scalar_type() == torch::kBFloat16) BY_D(short);
-  else {
-    TORCH_CHECK(q.scalar_type() == torch::kFloat32);
-    BY_D(float);
-  }
-#undef BY_D
+  if (DP == 32) PHASES(32);
+  else if (DP == 64) PHASES(64);
+  else if (DP == 128) PHASES(128);
+  else PHASES(256);
 #undef PHASES
   HIP_CHECK_LAST();
 }

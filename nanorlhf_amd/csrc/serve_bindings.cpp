@@ -25,7 +25,8 @@ void paged_attn_plain(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch
 void linear_attn_chunked(torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor pw,
                          OptTensor cs, bool interleaved, bool silu, double kscale,
                          torch::Tensor chunks, torch::Tensor first, torch::Tensor slots,
-                         torch::Tensor fresh, torch::Tensor state, torch::Tensor o);
+                         torch::Tensor fresh, torch::Tensor state, OptTensor gate, double eps,
+                         torch::Tensor o);
 void linear_attn_decode(torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor pw,
                         OptTensor cs, bool interleaved, bool silu, double kscale,
                         torch::Tensor slots, torch::Tensor seq_lens, torch::Tensor state,

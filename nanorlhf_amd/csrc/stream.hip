@@ -105,6 +105,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
     const T* __restrict__ in, const T* __restrict__ w, const T* __restrict__ gate,
     T* __restrict__ out, long units, int groups, int part, long ldg, long ldo, float eps) {
   constexpr int NT = NW * 64;
+  constexpr int REG = 2;          // vectors kept in registers between the passes
   __shared__ float scratch[4];
   const long unit = NW == 1 ? blockIdx.x * 4L + (threadIdx.x >> 6) : (long)blockIdx.x;
   if (unit >= units) return;
@@ -113,8 +114,18 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
   const long col = (unit % groups) * part;
   const T* src = in + row * (long)groups * part + col;
   const int nvec = part / VEC;
+  float keep[REG][VEC], kg[REG][VEC];
   float ss = 0.f;
-  for (int i = tid; i < nvec; i += NT) {
+#pragma unroll
+  for (int r = 0; r < REG; r++) {
+    const int i = tid + r * NT;
+    if (i >= nvec) break;
+    ldv<VEC>(src + (long)i * VEC, keep[r]);
+    ldv<VEC>(gate + row * ldg + col + (long)i * VEC, kg[r]);
+#pragma unroll
+    for (int j = 0; j < VEC; j++) ss += keep[r][j] * keep[r][j];
+  }
+  for (int i = tid + REG * NT; i < nvec; i += NT) {
     float v[VEC];
     ldv<VEC>(src + (long)i * VEC, v);
 #pragma unroll
@@ -122,10 +133,8 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
   }
   ss = unit_sum<NW>(ss, scratch);
   const float inv = 1.f / sqrtf(ss / (float)part + eps);
-  for (int i = tid; i < nvec; i += NT) {
-    float v[VEC], gv[VEC], wv[VEC];
-    ldv<VEC>(src + (long)i * VEC, v);
-    ldv<VEC>(gate + row * ldg + col + (long)i * VEC, gv);
+  auto emit = [&](int i, float* v, const float* gv) {
+    float wv[VEC];
     if (w) ldv<VEC>(w + col + (long)i * VEC, wv);
 #pragma unroll
     for (int j = 0; j < VEC; j++) {
@@ -133,6 +142,17 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
       v[j] = v[j] * inv * (w ? wv[j] : 1.f) * a;
     }
     stv<VEC>(out + row * ldo + col + (long)i * VEC, v);
+  };
+#pragma unroll
+  for (int r = 0; r < REG; r++) {
+    const int i = tid + r * NT;
+    if (i < nvec) emit(i, keep[r], kg[r]);
+  }
+  for (int i = tid + REG * NT; i < nvec; i += NT) {
+    float v[VEC], gv[VEC];
+    ldv<VEC>(src + (long)i * VEC, v);
+    ldv<VEC>(gate + row * ldg + col + (long)i * VEC, gv);
+    emit(i, v, gv);
   }
 }
 
@@ -184,102 +204,124 @@ __global__ __launch_bounds__(256) void rope_angles_kernel(
 }
 
 // ------------------------------------- rotary attention: q, k, v in one go
-// One wave per (token, head) of q, k and v, read from columns of the layer's
-// projection row:
+// Read from columns of the layer's projection row:
 //   q, k: RMS norm over the head with weight qw/kw (null: no norm), then
 //         rotation of the first rdims dimensions by csk;
 //   v:    rotation over all its dimensions by csv (null: none).
 // q goes to qo [T, H, DKP] (pad columns zeroed); k and v go straight into
 // their pages, K [P, ps, G, DKP], V [P, G, DVP, ps].  Pad columns of the pages
 // stay zero from the pool's creation.
+//
+// The first blocks take q and k: DKP / 4 lanes per (token, head), four
+// elements each.  The rest take v, 16 tokens of one head per block: rows in,
+// turned around in LDS, and out with tokens fastest, as the d-major pages want.
+struct QkvArgs {
+  long ld;
+  int qoff, koff, voff, H, G, D, V, DKP, DVP, rdims, interleaved, ps;
+  float eps;
+  const float *csk, *csv;
+  const long* slots;
+  long tokens, qk_blocks;
+};
+
+// two neighbouring elements (even offset)
+DEVINL void ld2(const short* p, float* o) {
+  const unsigned u = *reinterpret_cast<const unsigned*>(p);
+  o[0] = bf2f((short)(u & 0xffff));
+  o[1] = bf2f((short)(u >> 16));
+}
+DEVINL void ld2(const float* p, float* o) {
+  o[0] = p[0];
+  o[1] = p[1];
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void rotary_qkv_kernel(
-    const T* __restrict__ proj, long ld, int qoff, int koff, int voff,
-    const T* __restrict__ qw, const T* __restrict__ kw,
-    const float* __restrict__ csk, const float* __restrict__ csv,
-    const long* __restrict__ slots, T* __restrict__ qo, T* __restrict__ kc,
-    T* __restrict__ vc, long tokens, int H, int G, int D, int V, int DKP, int DVP,
-    int rdims, int interleaved, int ps, float eps) {
-  __shared__ float buf[4][256];
-  const int lane = threadIdx.x & 63;
-  float* wb = buf[threadIdx.x >> 6];
-  const int heads = H + 2 * G;
-  const long unit = blockIdx.x * 4L + (threadIdx.x >> 6);
-  if (unit >= tokens * heads) return;
-  const long t = unit / heads;
-  const int h = (int)(unit % heads);
-  const bool is_q = h < H, is_v = h >= H + G;
-  const int n = is_v ? V : D;
-  const int rot = is_v ? (csv ? V : 0) : rdims;
-  const float* cs = is_v ? csv + t * V : csk + t * (long)rdims;
-  const T* src = proj + t * ld +
-                 (is_q ? qoff + h * D : is_v ? voff + (h - H - G) * V : koff + (h - H) * D);
-  float x[4];
-  float ss = 0.f;
+    const T* __restrict__ proj, const T* __restrict__ qw, const T* __restrict__ kw,
+    T* __restrict__ qo, T* __restrict__ kc, T* __restrict__ vc, QkvArgs a) {
+  __shared__ float buf[16 * 257];
+  if (blockIdx.x < a.qk_blocks) {
+    const int lpu = a.DKP / 4;                      // lanes per unit: 8..64
+    const int heads = a.H + a.G;
+    const long unit = (long)blockIdx.x * (256 / lpu) + threadIdx.x / lpu;
+    if (unit >= a.tokens * heads) return;           // whole units leave together
+    const long t = unit / heads;
+    const int h = (int)(unit % heads);
+    const bool is_q = h < a.H;
+    const int e0 = 4 * (threadIdx.x % lpu);
+    const int D = a.D;
+    const T* src = proj + t * a.ld + (is_q ? a.qoff + h * D : a.koff + (h - a.H) * D);
+    const T* w = is_q ? qw : kw;
+    float x[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int r = 0; r < 2; r++) {
-    const int e = 2 * lane + 128 * r;
-    x[2 * r] = e < n ? ldf(src + e) : 0.f;
-    x[2 * r + 1] = e + 1 < n ? ldf(src + e + 1) : 0.f;
-    ss += x[2 * r] * x[2 * r] + x[2 * r + 1] * x[2 * r + 1];
-  }
-  const T* w = is_v ? nullptr : is_q ? qw : kw;
-  if (w) {
-    ss = wave_sum(ss);
-    const float inv = 1.f / sqrtf(ss / (float)n + eps);
+    for (int r = 0; r < 4; r += 2)
+      if (e0 + r < D) ld2(src + e0 + r, x + r);     // D is even
+    if (w) {
+      float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+      for (int off = lpu / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
+      const float inv = 1.f / sqrtf(ss / (float)D + a.eps);
 #pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int e = 2 * lane + 128 * (r >> 1) + (r & 1);
-      if (e < n) x[r] = x[r] * inv * ldf(w + e);
+      for (int r = 0; r < 4; r += 2)
+        if (e0 + r < D) {
+          float wv[2];
+          ld2(w + e0 + r, wv);
+          x[r] *= inv * wv[0];
+          x[r + 1] *= inv * wv[1];
+        }
     }
-  }
-  const int half = rot >> 1;
-  if (interleaved) {
+    const int half = a.rdims >> 1;
+    const float* cs = a.csk + t * (long)a.rdims;
+    if (a.interleaved) {
 #pragma unroll
-    for (int r = 0; r < 2; r++) {
-      const int p = lane + 64 * r;
-      if (p < half) {
-        const float c = cs[p], s = cs[half + p];
-        const float u = x[2 * r], v = x[2 * r + 1];
-        x[2 * r] = u * c - v * s;
-        x[2 * r + 1] = v * c + u * s;
+      for (int r = 0; r < 4; r += 2) {
+        const int p = (e0 + r) >> 1;
+        if (p < half) {
+          const float c = cs[p], s = cs[half + p], u = x[r], v = x[r + 1];
+          x[r] = u * c - v * s;
+          x[r + 1] = v * c + u * s;
+        }
+      }
+    } else if (half) {
+      float* ub = buf + (threadIdx.x / lpu) * (a.DKP + 1);   // 256 / lpu units fit
+#pragma unroll
+      for (int r = 0; r < 4; r++) ub[e0 + r] = x[r];
+      lds_fence_wave_kv();                           // a unit never spans waves
+#pragma unroll
+      for (int r = 0; r < 4; r++) {
+        const int e = e0 + r;
+        if (e < half) x[r] = x[r] * cs[e] - ub[e + half] * cs[half + e];
+        else if (e < a.rdims) x[r] = x[r] * cs[e - half] + ub[e - half] * cs[e];
       }
     }
-  } else if (rot) {
-#pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int e = 2 * lane + 128 * (r >> 1) + (r & 1);
-      if (e < n) wb[e] = x[r];
-    }
-    lds_fence_wave_kv();
-#pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int e = 2 * lane + 128 * (r >> 1) + (r & 1);
-      if (e < half) x[r] = x[r] * cs[e] - wb[e + half] * cs[half + e];
-      else if (e < rot) x[r] = x[r] * cs[e - half] + wb[e - half] * cs[e];
-    }
-  }
-  if (is_q) {
-    T* dst = qo + (t * H + h) * (long)DKP;
-#pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int e = 2 * lane + 128 * (r >> 1) + (r & 1);
-      if (e < DKP) stf(dst + e, e < n ? x[r] : 0.f);
-    }
+    T* dst = is_q ? qo + (t * a.H + h) * (long)a.DKP
+                  : kc + (a.slots[t] * a.G + (h - a.H)) * (long)a.DKP;
+    stv<4>(dst + e0, x);                             // pad elements are 0
     return;
   }
-  const long slot = slots[t];
-  const long page = slot / ps;
-  const int off = (int)(slot % ps);
-#pragma unroll
-  for (int r = 0; r < 4; r++) {
-    const int e = 2 * lane + 128 * (r >> 1) + (r & 1);
-    if (e >= n) continue;
-    if (is_v)
-      stf(vc + ((page * G + (h - H - G)) * (long)DVP + e) * ps + off, x[r]);
-    else
-      stf(kc + (slot * G + (h - H)) * (long)DKP + e, x[r]);
+  const long vb = blockIdx.x - a.qk_blocks;
+  const long t0 = vb / a.G * 16;
+  const int g = (int)(vb % a.G), V = a.V, half = V >> 1;
+  const int n = (int)min(16L, a.tokens - t0);
+  for (int i = threadIdx.x; i < n * half; i += 256) {
+    const int j = i / half, p = i % half;
+    const T* src = proj + (t0 + j) * a.ld + a.voff + g * V;
+    const int ea = a.interleaved ? 2 * p : p, eb = a.interleaved ? 2 * p + 1 : p + half;
+    float u = ldf(src + ea), v = ldf(src + eb);
+    if (a.csv) {
+      const float c = a.csv[(t0 + j) * V + p], s = a.csv[(t0 + j) * V + half + p];
+      const float y = u * c - v * s;
+      v = v * c + u * s;
+      u = y;
+    }
+    buf[j * 257 + ea] = u;
+    buf[j * 257 + eb] = v;
   }
+  __syncthreads();
+  const int j = threadIdx.x & 15;
+  if (j >= n) return;
+  const long slot = a.slots[t0 + j];
+  T* dst = vc + (slot / a.ps * a.G + g) * (long)a.DVP * a.ps + slot % a.ps;
+  for (int e = threadIdx.x >> 4; e < V; e += 16) stf(dst + (long)e * a.ps, buf[j * 257 + e]);
 }
 
 // ======================================================== host wrappers ==
@@ -365,7 +407,11 @@ void gated_norm(torch::Tensor in, c10::optional<torch::Tensor> w, torch::Tensor 
                      ptr<T>(in), optr<T>(w), ptr<T>(gate), ptr<T>(out), units,         \
                      (int)groups, part, ldg, ldo, (float)eps)
 #define GNA(VEC, NW) do { if (act == 0) GN(VEC, NW, 0); else GN(VEC, NW, 1); } while (0)
+    const bool vec8 = vec && sizeof(T) == 2 && part % 8 == 0 && ldg % 8 == 0 && ldo % 8 == 0 &&
+                      aligned(gate.data_ptr(), 16) && aligned(out.data_ptr(), 16);
     if (!vec) GNA(1, 1);
+    else if (vec8 && part > 1024) GNA(8, 4);
+    else if (vec8) GNA(8, 1);
     else if (part > 512) GNA(4, 4);
     else GNA(4, 1);
 #undef GNA
@@ -442,17 +488,38 @@ torch::Tensor rotary_qkv(torch::Tensor proj, long qoff, long koff, long voff,
   for (auto& w : {qw, kw})
     if (w.has_value())
       TORCH_CHECK(w->is_contiguous() && w->numel() == D && w->scalar_type() == proj.scalar_type());
+  TORCH_CHECK(qoff % 2 == 0 && koff % 2 == 0 && proj.stride(0) % 2 == 0 &&
+              aligned(proj.data_ptr(), 8), "projection columns start at even offsets");
+  TORCH_CHECK(DKP == 32 || DKP == 64 || DKP == 128 || DKP == 256, "unsupported key width ", DKP);
   auto qo = torch::empty({T, H, (long)DKP}, proj.options());
   if (T == 0) return qo;
-  const long units = T * (H + 2 * G);
+  const long units = T * (H + G), per = 256 / (DKP / 4);
+  QkvArgs a{};
+  a.ld = proj.stride(0);
+  a.qoff = qoff;
+  a.koff = koff;
+  a.voff = voff;
+  a.H = H;
+  a.G = G;
+  a.D = D;
+  a.V = V;
+  a.DKP = DKP;
+  a.DVP = DVP;
+  a.rdims = rdims;
+  a.interleaved = interleaved;
+  a.ps = ps;
+  a.eps = eps;
+  a.csk = optr<float>(csk);
+  a.csv = optr<float>(csv);
+  a.slots = slots.data_ptr<long>();
+  a.tokens = T;
+  a.qk_blocks = (units + per - 1) / per;
+  const long grid = a.qk_blocks + (T + 15) / 16 * G;
+  auto stream = at::hip::getCurrentHIPStream();
   by_type(proj, [&](auto tag) {
-    using T = decltype(tag);
-    hipLaunchKernelGGL((rotary_qkv_kernel<T>), dim3((units + 3) / 4), dim3(256), 0,
-                       at::hip::getCurrentHIPStream(), ptr<T>(proj), proj.stride(0), (int)qoff,
-                       (int)koff, (int)voff, optr<T>(qw), optr<T>(kw), optr<float>(csk),
-                       optr<float>(csv), slots.data_ptr<long>(), ptr<T>(qo), ptr<T>(kc),
-                       ptr<T>(vc), (long)proj.size(0), (int)H, (int)G, (int)D, (int)V, DKP, DVP,
-                       (int)rdims, (int)interleaved, ps, (float)eps);
+    using E = decltype(tag);
+    hipLaunchKernelGGL((rotary_qkv_kernel<E>), dim3(grid), dim3(256), 0, stream, ptr<E>(proj),
+                       optr<E>(qw), optr<E>(kw), ptr<E>(qo), ptr<E>(kc), ptr<E>(vc), a);
   });
   HIP_CHECK_LAST();
   return qo;

@@ -55,12 +55,15 @@ class LinearMixer(nn.Module):
         q, k, v, g = (proj[:, cols[n][0]:cols[n][1]] for n in ("q", "k", "v", "g"))
         T, nd = proj.shape[0], ctx.n_decode
         if nd:
-            self.decode(q[:nd], k[:nd], v[:nd], g[:nd], ctx, state, out[:nd],
-                        self._kw(ctx, 0, nd))
+            kw = self._kw(ctx, 0, nd)
+            self.run(lambda **f: ops.linear_attn_decode(
+                q[:nd], k[:nd], v[:nd], self.decay, ctx.state_slots, ctx.seq_lens, state,
+                **kw, **f), g[:nd], out[:nd])
         if ctx.portions is not None:
-            o = ops.linear_attn_chunked(q[nd:], k[nd:], v[nd:], self.decay, ctx.portions,
-                                        state, **self._kw(ctx, nd, T))
-            self.finish(o, g[nd:], out[nd:])
+            kw = self._kw(ctx, nd, T)
+            self.run(lambda **f: ops.linear_attn_chunked(
+                q[nd:], k[nd:], v[nd:], self.decay, ctx.portions, state, **kw, **f),
+                g[nd:], out[nd:])
 
 
 class Retention(LinearMixer):
@@ -72,12 +75,8 @@ class Retention(LinearMixer):
         self.rotation = ops.Rotation(m["rot"]["dims"], m["rot"]["base"])
         self.kscale = self.dim ** -0.5
 
-    def decode(self, q, k, v, g, ctx, state, out, kw):
-        ops.linear_attn_decode(q, k, v, self.decay, ctx.state_slots, ctx.seq_lens, state,
-                               gate=g, eps=self.eps, out=out, **kw)
-
-    def finish(self, o, g, out):
-        ops.gated_norm(o, None, g, out, self.eps, groups=self.heads, act="silu")
+    def run(self, attn, g, out):
+        attn(gate=g, eps=self.eps, out=out)
 
 
 class Lightning(LinearMixer):
@@ -94,13 +93,8 @@ class Lightning(LinearMixer):
     def weights(self):
         return {"norm": self.norm}
 
-    def decode(self, q, k, v, g, ctx, state, out, kw):
-        o = ops.linear_attn_decode(q, k, v, self.decay, ctx.state_slots, ctx.seq_lens, state,
-                                   **kw)
-        self.finish(o, g, out)
-
-    def finish(self, o, g, out):
-        ops.gated_norm(o, self.norm, g, out, self.eps, act="sigmoid")
+    def run(self, attn, g, out):
+        ops.gated_norm(attn(), self.norm, g, out, self.eps, act="sigmoid")
 
 
 class WindowAttention(nn.Module):

@@ -14,9 +14,11 @@ from __future__ import annotations
 import torch
 
 from . import serve_ext
+from .rmsnorm import gated_norm
 from .rope import rotate_pairs
 
 CHUNK = 64
+FUSED_VDIM = 128      # widest head whose norm and gate fit the chunk kernel's epilogue
 
 
 class DecayTable:
@@ -48,17 +50,29 @@ def _inputs(q, k, v, H, cs, interleaved, silu, kscale):
 
 
 def linear_attn_chunked(q, k, v, decay: DecayTable, portions, state, *, cs=None,
-                        interleaved: bool = False, silu: bool = False,
-                        kscale: float = 1.0) -> torch.Tensor:
+                        interleaved: bool = False, silu: bool = False, kscale: float = 1.0,
+                        gate=None, eps: float = 0.0, out=None) -> torch.Tensor:
     """q, k [T, H*D], v [T, H*V]: the tokens of `portions` (packed).  Each
     portion goes on from its slot of state [slots, H, D, V] (from zero if it
-    starts its sequence) and leaves its last state there.  Returns [T, H*V]."""
-    o = torch.empty(v.shape, dtype=v.dtype, device=v.device)
+    starts its sequence) and leaves its last state there.  `gate` and `out` as
+    for linear_attn_decode."""
+    if out is None:
+        out = torch.empty(v.shape, dtype=v.dtype, device=v.device)
+    o = out
     if q.is_cuda:
+        fused = gate is not None and q.dtype == torch.bfloat16 \
+            and v.shape[1] // decay.heads <= FUSED_VDIM
+        if gate is not None and not fused:
+            o = torch.empty(v.shape, dtype=v.dtype, device=v.device)
         serve_ext().linear_attn_chunked(q, k, v, decay.on(q.device), cs, interleaved, silu,
                                         float(kscale), portions.chunks, portions.chunk_first,
-                                        portions.state_slots, portions.fresh, state, o)
-        return o
+                                        portions.state_slots, portions.fresh, state,
+                                        gate if fused else None, float(eps), o)
+        if gate is not None and not fused:
+            gated_norm(o, None, gate, out, eps, groups=decay.heads)
+        return out
+    if gate is not None:
+        o = torch.empty(v.shape, dtype=torch.float32)
     H, pw = decay.heads, decay.on("cpu")
     q, k, v = _inputs(q, k, v, H, cs, interleaved, silu, kscale)
     ch = portions.chunks
@@ -75,7 +89,9 @@ def linear_attn_chunked(q, k, v, decay: DecayTable, portions, state, *, cs=None,
             o[r:r + n] = (inside + ahead).transpose(0, 1).reshape(n, -1).to(o.dtype)
             S = pw[:, n, None, None] * S + (kk * pw[:, n - 1 - i, None]).transpose(1, 2) @ vv
         state[slot] = S
-    return o
+    if gate is not None:
+        gated_norm(o, None, gate, out, eps, groups=decay.heads)
+    return out
 
 
 def linear_attn_decode(q, k, v, decay: DecayTable, slots, seq_lens, state, *, cs=None,

@@ -1,0 +1,102 @@
+"""Serving throughput of Gonurax beside Qwen2 at equal size.
+
+Equal size: width, feed-forward, layers, vocabulary, and softmax heads of one
+width; Gonurax's linear-attention heads are as many and as wide as the query
+heads.  Prompts run through SamplerEngine's prefill, decoding through its
+captured decode step, both with bf16 caches and random weights."""
+from __future__ import annotations
+
+import json
+import time
+
+import torch
+
+from ..models import build_model
+from ..models.config import ModelConfig, _gonurax_layers
+from ..models.gonurax import GonuraxConfig
+from ..sampler import SamplerEngine, SamplingParams, SeqState
+from ..sampler.decode_batch import DecodeBatch
+
+VOCAB, LAYERS = 32768, 6
+#           width    ff  heads  kv
+SIZES = {
+    "1.5b": (1536, 8960, 12, 2),
+    "3b": (2048, 11008, 16, 2),
+    "8b": (4096, 14336, 32, 8),
+}
+PREFILL = [(8, 2048), (1, 16384)]     # prompts x tokens
+DECODE = [(256, 2048), (32, 2048)]    # sequences x context
+
+
+def make_config(model: str, size: str):
+    W, ff, H, G = SIZES[size]
+    if model == "qwen2":
+        return ModelConfig(vocab_size=VOCAB, hidden_size=W, num_layers=LAYERS, num_heads=H,
+                           num_kv_heads=G, head_dim=128, intermediate_size=ff,
+                           max_position=20000)
+    return GonuraxConfig(vocab_size=VOCAB, hidden_size=W, norm_groups=4, residual_mult=0.5,
+                         **_gonurax_layers(LAYERS, heads=H, dim=128, vdim=128, attn_heads=H,
+                                           kv_heads=G, attn_dim=128, ff=ff, window=1024,
+                                           keep_first=4))
+
+
+def _timed(fn, steps):
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / steps
+
+
+def measure(model: str, size: str, steps: int, warmup: int):
+    torch.manual_seed(0)
+    torch.set_default_dtype(torch.bfloat16)
+    m = build_model(make_config(model, size)).to("cuda").eval()
+    torch.set_default_dtype(torch.float32)
+    params = SamplingParams(temperature=1.0, top_p=0.95, max_tokens=4096)
+
+    def report(what, n, length, tokens, seconds):
+        print(json.dumps({"serving": what, "model": model, "size": size, "layers": LAYERS,
+                          "sequences": n, "length": length,
+                          "tokens_per_s": round(tokens / seconds),
+                          "ms": round(seconds * 1e3, 3)}), flush=True)
+
+    for n, length in PREFILL:
+        eng = SamplerEngine(m, kv_pool_tokens=n * (length + 16), state_slots=n,
+                            kv_cache_dtype="bf16")
+        prompts = torch.randint(2, VOCAB, (n, length)).tolist()
+
+        def prefill():
+            seqs = [SeqState(i, p, i) for i, p in enumerate(prompts)]
+            for s in seqs:
+                s.ensure_capacity(eng.pool, length + 1)
+            eng._prefill(seqs, params)
+            for s in seqs:
+                eng.pool.release(s)
+
+        _timed(prefill, warmup + 1)
+        report("prefill", n, length, n * length, _timed(prefill, max(steps, 3)))
+        del eng
+    for n, length in DECODE:
+        eng = SamplerEngine(m, kv_pool_tokens=n * (length + 512), state_slots=n,
+                            kv_cache_dtype="bf16")
+        seqs = [SeqState(i, [2] * length, i) for i in range(n)]
+        for s in seqs:
+            s.ensure_capacity(eng.pool, length + 256)
+        eng._step_dev.zero_()
+        db = DecodeBatch(eng.pool, seqs, params.max_tokens, None, eng.device)
+
+        def decode():
+            eng._run_decode_step(db, params)
+
+        _timed(decode, 4)        # eager warm-up steps, then the capture
+        report("decode", n, length, n, _timed(decode, 50))
+        del eng, db
+
+
+@torch.no_grad()
+def run(sizes: str, models, steps: int, warmup: int) -> None:
+    for size in (SIZES if sizes == "all" else sizes.split(",")):
+        for model in models:
+            measure(model, size, steps, warmup)
