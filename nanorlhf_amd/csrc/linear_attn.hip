@@ -312,43 +312,43 @@ DEVINL void load_runs(const short* row, int g, const Source& s, const float* cs,
 
 constexpr int TS = CHUNK + 8;    // LDS row of a [feature][token] tile
 
-// vt[e][j] = v_j[v0 + e], 0 past the chunk's tokens and past V
-template <int VB, int NT>
-DEVINL void stage_v(short* vt, const short* v, const Source& s, long t0, int n, int h, int v0,
-                    bool vec) {
-  for (int i = threadIdx.x; i < (CHUNK / 4) * (VB / 4); i += NT) {
-    const int e = (i % (VB / 4)) * 4, j = (i / (VB / 4)) * 4;
-    float x[4][4];
+// Four tokens by four columns of v, turned around for a tile vt[e][j] =
+// v_j[v0 + e]; 0 past the chunk's tokens and past V.
+template <int VB>
+struct VPatch {
+  static constexpr int COUNT = (CHUNK / 4) * (VB / 4);
+  s16x4 col[4];
+  int e, j;
+  DEVINL void load(int i, const short* v, const Source& s, long t0, int n, int h, int v0,
+                   bool vec) {
+    e = (i % (VB / 4)) * 4;
+    j = (i / (VB / 4)) * 4;
 #pragma unroll
     for (int r = 0; r < 4; r++) {
       const short* row = v + (t0 + j + r) * s.ld + h * s.V + v0 + e;
-#pragma unroll
-      for (int c = 0; c < 4; c++) x[r][c] = 0.f;
+      float x[4] = {0.f, 0.f, 0.f, 0.f};
       if (j + r < n) {
         if (vec) {
-          if (v0 + e < s.V) ldv<4>(row, x[r]);
+          if (v0 + e < s.V) ldv<4>(row, x);
         } else {
 #pragma unroll
           for (int c = 0; c < 4; c++)
-            if (v0 + e + c < s.V) x[r][c] = ldf(row + c);
+            if (v0 + e + c < s.V) x[c] = ldf(row + c);
         }
       }
-      if (s.silu) {
 #pragma unroll
-        for (int c = 0; c < 4; c++) x[r][c] = silu_fast(x[r][c]);
-      }
-    }
-#pragma unroll
-    for (int c = 0; c < 4; c++) {
-      const float col[4] = {x[0][c], x[1][c], x[2][c], x[3][c]};
-      stv<4>(vt + (e + c) * TS + j, col);
+      for (int c = 0; c < 4; c++) col[c][r] = f2bf(s.silu ? silu_fast(x[c]) : x[c]);
     }
   }
-}
+  DEVINL void store(short* vt) const {
+#pragma unroll
+    for (int c = 0; c < 4; c++) *reinterpret_cast<s16x4*>(vt + (e + c) * TS + j) = col[c];
+  }
+};
 
 // ws [chunks, H, V, DP]: what a chunk adds, feature-major
 template <int DP, int VB>
-__global__ __launch_bounds__(256) void chunk_state_split_kernel(
+__global__ __launch_bounds__(512) void chunk_state_split_kernel(
     const short* __restrict__ k, const short* __restrict__ v, Source s, Chunks ch,
     const float* __restrict__ pw, float* __restrict__ ws, bool vec) {
   __shared__ __attribute__((aligned(16))) short kt[2][DP * TS], vt[VB * TS];
@@ -356,8 +356,14 @@ __global__ __launch_bounds__(256) void chunk_state_split_kernel(
   const int n = ch.len[c];
   const long t0 = ch.row[c];
   const float* pwh = pw + h * (CHUNK + 1);
-  stage_v<VB, 256>(vt, v, s, t0, n, h, v0, vec);
-  for (int i = threadIdx.x; i < (CHUNK / 4) * (DP / 8); i += 256) {
+  // one half of the workgroup stages v, the other k
+  if (threadIdx.x >= 256) {
+    for (int i = threadIdx.x - 256; i < VPatch<VB>::COUNT; i += 256) {
+      VPatch<VB> x;
+      x.load(i, v, s, t0, n, h, v0, vec);
+      x.store(vt);
+    }
+  } else for (int i = threadIdx.x; i < (CHUNK / 4) * (DP / 8); i += 256) {
     const int g = i % (DP / 8), j = (i / (DP / 8)) * 4;
     float a[4][4], b[4][4];
     int ea = 8 * g, eb = ea + 4;
@@ -389,33 +395,24 @@ __global__ __launch_bounds__(256) void chunk_state_split_kernel(
   __syncthreads();
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lo = lane & 15, hi = lane >> 4;
-  constexpr int CW = VB / 64;                  // v tiles per wave
-  bf16x8l vf[CW][2];
+  constexpr int CT = VB / 16;                  // v tiles: 4 or 8
+  constexpr int RW = DP / 16 * CT / 8;         // feature tiles per wave
+  const int ct = w % CT, r0 = (w / CT) * RW;
+  bf16x8l vf[2];
 #pragma unroll
-  for (int q = 0; q < CW; q++)
+  for (int ks = 0; ks < 2; ks++) vf[ks] = frag(&vt[(ct * 16 + lo) * TS + 32 * ks + 8 * hi]);
+  const int e = v0 + ct * 16 + lo;
+  float* u = ws + (((long)c * s.H + h) * s.V + e) * DP;
+#pragma unroll 4
+  for (int rt = r0; rt < r0 + RW; rt++) {
+    f32x4 acc{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int ks = 0; ks < 2; ks++)
-      vf[q][ks] = frag(&vt[((w * CW + q) * 16 + lo) * TS + 32 * ks + 8 * hi]);
-  float* u = ws + ((long)c * s.H + h) * s.V * DP;
-#pragma unroll 2
-  for (int rt = 0; rt < DP / 16; rt++) {
-    bf16x8l kf[2][2];
-#pragma unroll
-    for (int pl = 0; pl < 2; pl++)
-#pragma unroll
-      for (int ks = 0; ks < 2; ks++)
-        kf[pl][ks] = frag(&kt[pl][(16 * rt + lo) * TS + 32 * ks + 8 * hi]);
-#pragma unroll
-    for (int q = 0; q < CW; q++) {
-      f32x4 acc{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ks = 0; ks < 2; ks++) {
-        acc = mfma16l(kf[1][ks], vf[q][ks], acc);
-        acc = mfma16l(kf[0][ks], vf[q][ks], acc);
-      }
-      const int e = v0 + (w * CW + q) * 16 + lo;
-      if (e < s.V) *reinterpret_cast<f32x4*>(u + (long)e * DP + 16 * rt + 4 * hi) = acc;
+    for (int ks = 0; ks < 2; ks++) {
+      const int at = (16 * rt + lo) * TS + 32 * ks + 8 * hi;
+      acc = mfma16l(frag(&kt[1][at]), vf[ks], acc);
+      acc = mfma16l(frag(&kt[0][at]), vf[ks], acc);
     }
+    if (e < s.V) *reinterpret_cast<f32x4*>(u + 16 * rt + 4 * hi) = acc;
   }
 }
 
@@ -458,19 +455,21 @@ __global__ __launch_bounds__(256) void chunk_scan_split_kernel(
 // transposed (a lane holds one token's consecutive columns).  With a gate (V
 // <= VB), the head's output leaves normed and gated.
 template <int DP, int VB>
-__global__ __launch_bounds__(512) void chunk_out_split_kernel(
+__global__ __launch_bounds__(512, DP > 128 ? 2 : 4) void chunk_out_split_kernel(
     const short* __restrict__ q, const short* __restrict__ k, const short* __restrict__ v,
     Source s, Chunks ch, const float* __restrict__ pw, const unsigned* __restrict__ ws,
     const short* __restrict__ gate, long ldg, float eps, short* __restrict__ o, long ldo,
     bool vec) {
   constexpr int QS = DP + 8;
-  constexpr int KR = 2 * CHUNK * (QS > TS ? QS : TS);
+  constexpr int PV = 2 * CHUNK * TS + VB * TS;
+  constexpr int KR = 2 * CHUNK * QS > PV ? 2 * CHUNK * QS : PV;
   constexpr int CT = VB / 16;             // v tiles: 4 or 8
   constexpr int RW = CT / 2;              // token tiles per wave
-  __shared__ __attribute__((aligned(16))) short qt[2][CHUNK * QS], kreg[KR], vt[VB * TS];
+  __shared__ __attribute__((aligned(16))) short qt[2][CHUNK * QS], kreg[KR];
   __shared__ float pws[CHUNK + 1], red[CT][CHUNK];
   short* kt[2] = {kreg, kreg + CHUNK * QS};
-  short* pt[2] = {kreg, kreg + CHUNK * TS};    // scores take the keys' place
+  short* pt[2] = {kreg, kreg + CHUNK * TS};    // scores and v take the keys' place
+  short* vt = kreg + 2 * CHUNK * TS;
   const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
   const int n = ch.len[c];
   const long t0 = ch.row[c];
@@ -501,7 +500,8 @@ __global__ __launch_bounds__(512) void chunk_out_split_kernel(
     *reinterpret_cast<s16x4*>(&kt[0][j * QS + eb]) = hi;
     *reinterpret_cast<s16x4*>(&kt[1][j * QS + eb]) = lo;
   }
-  stage_v<VB, 512>(vt, v, s, t0, n, h, v0, vec);
+  VPatch<VB> vp;
+  if (threadIdx.x < VPatch<VB>::COUNT) vp.load(threadIdx.x, v, s, t0, n, h, v0, vec);
   __syncthreads();
 
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -557,6 +557,7 @@ __global__ __launch_bounds__(512) void chunk_out_split_kernel(
     }
   }
   __syncthreads();                 // every wave is done with the keys
+  if (threadIdx.x < VPatch<VB>::COUNT) vp.store(vt);
 #pragma unroll
   for (int x = 0; x < 2; x++) {
     const int i = 16 * it + lo, j = 16 * (jt + x) + 4 * hi;
@@ -773,7 +774,7 @@ void linear_attn_chunked(torch::Tensor q, torch::Tensor k, torch::Tensor v, torc
 #define SPLIT(DD, VB)                                                                           \
   do {                                                                                          \
     const dim3 sg(n, s.H, (s.V + VB - 1) / VB);                                                 \
-    hipLaunchKernelGGL((chunk_state_split_kernel<DD, VB>), sg, dim3(256), 0, stream,            \
+    hipLaunchKernelGGL((chunk_state_split_kernel<DD, VB>), sg, dim3(512), 0, stream,            \
                        (const short*)k.data_ptr(), (const short*)v.data_ptr(), s, ch, pwp, wsp, \
                        vec);                                                                    \
     hipLaunchKernelGGL(chunk_scan_split_kernel, dim3(B, s.H, (s.V * DD + 255) / 256),           \

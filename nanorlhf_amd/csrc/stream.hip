@@ -212,12 +212,13 @@ __global__ __launch_bounds__(256) void rope_angles_kernel(
 // their pages, K [P, ps, G, DKP], V [P, G, DVP, ps].  Pad columns of the pages
 // stay zero from the pool's creation.
 //
-// The first blocks take q and k: DKP / 4 lanes per (token, head), four
+// The first blocks take q and k: DKP / 8 lanes per (token, head), eight
 // elements each.  The rest take v, 16 tokens of one head per block: rows in,
 // turned around in LDS, and out with tokens fastest, as the d-major pages want.
 struct QkvArgs {
   long ld;
   int qoff, koff, voff, H, G, D, V, DKP, DVP, rdims, interleaved, ps;
+  int tpb, vec;             // tokens per q/k block; heads load as 8-element vectors
   float eps;
   const float *csk, *csv;
   const long* slots;
@@ -241,61 +242,85 @@ __global__ __launch_bounds__(256) void rotary_qkv_kernel(
     T* __restrict__ qo, T* __restrict__ kc, T* __restrict__ vc, QkvArgs a) {
   __shared__ float buf[16 * 257];
   if (blockIdx.x < a.qk_blocks) {
-    const int lpu = a.DKP / 4;                      // lanes per unit: 8..64
-    const int heads = a.H + a.G;
-    const long unit = (long)blockIdx.x * (256 / lpu) + threadIdx.x / lpu;
-    if (unit >= a.tokens * heads) return;           // whole units leave together
-    const long t = unit / heads;
-    const int h = (int)(unit % heads);
-    const bool is_q = h < a.H;
-    const int e0 = 4 * (threadIdx.x % lpu);
-    const int D = a.D;
-    const T* src = proj + t * a.ld + (is_q ? a.qoff + h * D : a.koff + (h - a.H) * D);
-    const T* w = is_q ? qw : kw;
-    float x[4] = {0.f, 0.f, 0.f, 0.f};
+    const int lpu = a.DKP / 8;                      // lanes per unit: 4..32
+    const int heads = a.H + a.G, D = a.D, half = a.rdims >> 1;
+    const long tb = (long)blockIdx.x * a.tpb;
+    const int units = (int)min((long)a.tpb, a.tokens - tb) * heads;
+    const int e0 = 8 * (threadIdx.x % lpu);
+    float wq[8] = {}, wk[8] = {};                   // this lane's norm weights
+    if (qw)
 #pragma unroll
-    for (int r = 0; r < 4; r += 2)
-      if (e0 + r < D) ld2(src + e0 + r, x + r);     // D is even
-    if (w) {
-      float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
-      for (int off = lpu / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
-      const float inv = 1.f / sqrtf(ss / (float)D + a.eps);
-#pragma unroll
-      for (int r = 0; r < 4; r += 2)
+      for (int r = 0; r < 8; r += 2)
         if (e0 + r < D) {
-          float wv[2];
-          ld2(w + e0 + r, wv);
-          x[r] *= inv * wv[0];
-          x[r + 1] *= inv * wv[1];
+          ld2(qw + e0 + r, wq + r);
+          ld2(kw + e0 + r, wk + r);
         }
-    }
-    const int half = a.rdims >> 1;
-    const float* cs = a.csk + t * (long)a.rdims;
-    if (a.interleaved) {
+    // every unit's lanes stay together: units is the same for a whole block
+    for (int un = threadIdx.x / lpu; un < units; un += 256 / lpu) {
+      const long t = tb + un / heads;
+      const int h = un % heads;
+      const bool is_q = h < a.H;
+      const T* src = proj + t * a.ld + (is_q ? a.qoff + h * D : a.koff + (h - a.H) * D);
+      float x[8] = {};
+      if (a.vec) {
+        if (e0 < D) ldv<8>(src + e0, x);
+      } else {
 #pragma unroll
-      for (int r = 0; r < 4; r += 2) {
-        const int p = (e0 + r) >> 1;
-        if (p < half) {
-          const float c = cs[p], s = cs[half + p], u = x[r], v = x[r + 1];
-          x[r] = u * c - v * s;
-          x[r + 1] = v * c + u * s;
+        for (int r = 0; r < 8; r += 2)
+          if (e0 + r < D) ld2(src + e0 + r, x + r);   // D is even
+      }
+      const float* cs = a.csk + t * (long)a.rdims;
+      float c4[4], s4[4];                            // of four interleaved pairs
+      if (a.interleaved) {
+        const int p = e0 >> 1;
+        if (a.vec) {
+          if (p < half) {
+            ldv<4>(cs + p, c4);
+            ldv<4>(cs + half + p, s4);
+          }
+        } else {
+#pragma unroll
+          for (int r = 0; r < 4; r++)
+            if (p + r < half) {
+              c4[r] = cs[p + r];
+              s4[r] = cs[half + p + r];
+            }
         }
       }
-    } else if (half) {
-      float* ub = buf + (threadIdx.x / lpu) * (a.DKP + 1);   // 256 / lpu units fit
+      if (qw) {
+        float ss = 0.f;
 #pragma unroll
-      for (int r = 0; r < 4; r++) ub[e0 + r] = x[r];
-      lds_fence_wave_kv();                           // a unit never spans waves
+        for (int r = 0; r < 8; r++) ss += x[r] * x[r];
+        for (int off = lpu / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
+        const float inv = 1.f / sqrtf(ss / (float)D + a.eps);
 #pragma unroll
-      for (int r = 0; r < 4; r++) {
-        const int e = e0 + r;
-        if (e < half) x[r] = x[r] * cs[e] - ub[e + half] * cs[half + e];
-        else if (e < a.rdims) x[r] = x[r] * cs[e - half] + ub[e - half] * cs[e];
+        for (int r = 0; r < 8; r++) x[r] *= inv * (is_q ? wq[r] : wk[r]);
       }
+      if (a.interleaved) {
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+          if ((e0 >> 1) + r < half) {
+            const float u = x[2 * r], v = x[2 * r + 1];
+            x[2 * r] = u * c4[r] - v * s4[r];
+            x[2 * r + 1] = v * c4[r] + u * s4[r];
+          }
+      } else if (half) {
+        float* ub = buf + (threadIdx.x / lpu) * (a.DKP + 1);   // 256 / lpu units fit
+#pragma unroll
+        for (int r = 0; r < 8; r++) ub[e0 + r] = x[r];
+        lds_fence_wave_kv();                         // a unit never spans waves
+#pragma unroll
+        for (int r = 0; r < 8; r++) {
+          const int e = e0 + r;
+          if (e < half) x[r] = x[r] * cs[e] - ub[e + half] * cs[half + e];
+          else if (e < a.rdims) x[r] = x[r] * cs[e - half] + ub[e - half] * cs[e];
+        }
+        lds_fence_wave_kv();                         // before the next unit's stores
+      }
+      T* dst = is_q ? qo + (t * a.H + h) * (long)a.DKP
+                    : kc + (a.slots[t] * a.G + (h - a.H)) * (long)a.DKP;
+      stv<8>(dst + e0, x);                           // pad elements are 0
     }
-    T* dst = is_q ? qo + (t * a.H + h) * (long)a.DKP
-                  : kc + (a.slots[t] * a.G + (h - a.H)) * (long)a.DKP;
-    stv<4>(dst + e0, x);                             // pad elements are 0
     return;
   }
   const long vb = blockIdx.x - a.qk_blocks;
@@ -485,6 +510,7 @@ torch::Tensor rotary_qkv(torch::Tensor proj, long qoff, long koff, long voff,
   if (csv.has_value())
     TORCH_CHECK(csv->is_contiguous() && csv->size(0) == T && csv->size(1) == V &&
                 csv->scalar_type() == torch::kFloat32);
+  TORCH_CHECK(qw.has_value() == kw.has_value());
   for (auto& w : {qw, kw})
     if (w.has_value())
       TORCH_CHECK(w->is_contiguous() && w->numel() == D && w->scalar_type() == proj.scalar_type());
@@ -493,7 +519,7 @@ torch::Tensor rotary_qkv(torch::Tensor proj, long qoff, long koff, long voff,
   TORCH_CHECK(DKP == 32 || DKP == 64 || DKP == 128 || DKP == 256, "unsupported key width ", DKP);
   auto qo = torch::empty({T, H, (long)DKP}, proj.options());
   if (T == 0) return qo;
-  const long units = T * (H + G), per = 256 / (DKP / 4);
+  const long per = 256 / (DKP / 8);
   QkvArgs a{};
   a.ld = proj.stride(0);
   a.qoff = qoff;
@@ -513,7 +539,12 @@ torch::Tensor rotary_qkv(torch::Tensor proj, long qoff, long koff, long voff,
   a.csv = optr<float>(csv);
   a.slots = slots.data_ptr<long>();
   a.tokens = T;
-  a.qk_blocks = (units + per - 1) / per;
+  // several units per thread once there are blocks enough to fill the chip
+  a.tpb = std::max<long>(1, per * (T * (H + G) / per > 8192 ? 4 : 1) / (H + G));
+  a.vec = D % 8 == 0 && rdims % 8 == 0 && aligned(a.csk, 16) && qoff % 8 == 0 &&
+          koff % 8 == 0 && a.ld % 8 == 0 &&
+          aligned(proj.data_ptr(), 16);
+  a.qk_blocks = (T + a.tpb - 1) / a.tpb;
   const long grid = a.qk_blocks + (T + 15) / 16 * G;
   auto stream = at::hip::getCurrentHIPStream();
   by_type(proj, [&](auto tag) {
