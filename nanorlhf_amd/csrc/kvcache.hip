@@ -201,7 +201,7 @@ __global__ void paged_decode_kernel(const short* __restrict__ q,    // [B, Hq, D
   // On the fp8 cache path Q is quantized to e4m3 once here and the QK^T
   // runs on mfma_f32_16x16x32_fp8_fp8 — K-cache bytes feed the MFMA
   // directly (no dequant pass), doubling matrix throughput on top of the
-  // halved KV stream (VERDICT #9 / ROADMAP #4).
+  // halved KV stream.
   constexpr bool FP8 = sizeof(CT) == 1;
   bf16x8k qf[NC];
   long qf8[NC];

@@ -46,7 +46,7 @@ __global__ void sample_topp_kernel(const LT* __restrict__ logits,
   const int nvec = V / 8;
 
   // ---- pass 1: plain row max + argmax ----------------------------------
-  // (the round-1 online (m,s) update carried m,s ACROSS loop iterations —
+  // (an online (m,s) update would carry m,s ACROSS loop iterations —
   // a serial exp/fma dependency chain per wave; plain fmax has none, and
   // the exp-sum folds into the histogram pass below, which also drops one
   // full read of the row)

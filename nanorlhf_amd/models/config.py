@@ -1,7 +1,6 @@
 """Model configurations and named presets.
 
-Presets cover the model families the reference runs (SURVEY.md §6 /
-BASELINE.json configs): Qwen2.5-{0.5,1.5,7}B policy shapes, a
+Presets cover the model families the reference runs: Qwen2.5-{0.5,1.5,7}B policy shapes, a
 deberta-v3-large-SHAPED bidirectional reward encoder (same parameter count /
 layer geometry; MI355X-native architecture, not a DeBERTa port), and the
 2-layer 128-dim tiny model for the CPU plumbing config."""
@@ -74,7 +73,7 @@ def _gonurax_layers(n, *, heads, dim, vdim, attn_heads, kv_heads, attn_dim, ff, 
 
 
 PRESETS: dict[str, dict] = {
-    # BASELINE config #1: 2-layer 128-dim tiny model, CPU-only plumbing.
+    # 2-layer 128-dim tiny model, CPU-only plumbing.
     "tiny": dict(vocab_size=1024, hidden_size=128, num_layers=2, num_heads=4,
                  num_kv_heads=2, head_dim=32, intermediate_size=512,
                  max_position=2048, rope_theta=1e4, dtype="float32"),

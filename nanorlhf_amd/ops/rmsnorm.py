@@ -1,7 +1,6 @@
 """RMSNorm forward/backward.
 
-Replaces transformers' Qwen2RMSNorm used inside every reference model call
-(SURVEY.md §2.2 row "RMSNorm, RoPE, SwiGLU").  GPU path is a fused HIP
+Replaces transformers' Qwen2RMSNorm used inside every reference model call.  GPU path is a fused HIP
 kernel (one pass, bf16x8 vector loads, fp32 accumulation)."""
 from __future__ import annotations
 

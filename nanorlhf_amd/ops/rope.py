@@ -1,8 +1,7 @@
 """Rotary position embedding (NeoX rotate-half layout, Qwen2 semantics).
 
 cos/sin tables are precomputed on host once per model (fp32, [max_pos, D/2])
-— on-device trig would turn this memory-bound op VALU-bound
-(cdna_hip_programming.md Appendix B).  The HIP kernel applies RoPE in place
+— on-device trig would turn this memory-bound op VALU-bound.  The HIP kernel applies RoPE in place
 to q and k with a sign flag so backward reuses the same kernel with sin
 negated (rotation transpose)."""
 from __future__ import annotations

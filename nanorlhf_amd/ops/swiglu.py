@@ -1,6 +1,6 @@
 """Fused SwiGLU activation: y = silu(gate) * up, with gate/up interleaved as
 one [N, 2*I] tensor (the gate_up projection's output).  Fusing halves the
-HBM round-trips vs separate silu+mul (SURVEY.md §2.2)."""
+HBM round-trips vs separate silu+mul."""
 from __future__ import annotations
 
 import torch

@@ -273,6 +273,55 @@ def test_attention(dev, dtype, tol, dims, mask, rot, sizes):
 
 
 @kinds
+@pytest.mark.parametrize("D,V,rot", [(24, 20, 16), (64, 32, 64), (130, 34, 2), (10, 6, 6)])
+def test_rotate_half_layout_of_q_k_v(dev, dtype, tol, D, V, rot):
+    """The other layout of pairs through the same preparation step."""
+    H, G, T = 3, 1, 37
+    x = rand(T, (H + G) * D + G * V, seed=4, dtype=dtype)
+    DP, VP = ops.pad_head_dim(D), ops.pad_head_dim(V)
+    kc = torch.zeros(4, 16, G, DP, dtype=dtype, device=dev)
+    vc = torch.zeros(4, G, VP, 16, dtype=dtype, device=dev)
+    pos = torch.arange(3, 3 + T)
+    slots = torch.arange(T - 1, -1, -1) + 5
+    rk, rv = ops.Rotation(rot, 90.0), ops.Rotation(V, 90.0)
+    q = ops.rotary_qkv(x.to(dev), (0, H * D, (H + G) * D), H, G, D, V, slots.to(dev), kc, vc,
+                       cs_qk=rk.angles(pos.to(dev)), cs_v=rv.angles(pos.to(dev)))
+    xd = x.double()
+    want_q = orc.rotate_half(xd[:, :H * D].view(T, H, D), pos, 90.0, rot)
+    want_k = orc.rotate_half(xd[:, H * D:(H + G) * D].view(T, G, D), pos, 90.0, rot)
+    want_v = orc.rotate_half(xd[:, (H + G) * D:].view(T, G, V), pos, 90.0, V)
+    close(q[..., :D], want_q, tol)
+    close(kc.cpu()[slots // 16, slots % 16, :, :D], want_k, tol)
+    close(vc.cpu()[slots // 16, :, :V, slots % 16], want_v, tol)
+    assert q[..., D:].abs().sum() == 0 and kc[..., D:].abs().sum() == 0
+    assert vc[:, :, V:].abs().sum() == 0
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("interleaved", [True, False])
+def test_qkv_of_a_large_batch_equals_its_parts(dtype, interleaved):
+    H, G, D, V, T, dev = 7, 2, 200, 96, 8192, "cuda"
+    x = rand(T, (H + G) * D + G * V, seed=6, dtype=dtype).to(dev)
+    w = tuple((1 + rand(D, seed=s) / 4).to(dtype).to(dev) for s in (1, 2))
+    pos = torch.arange(T, device=dev)
+    ck = ops.Rotation(192, 5e3, interleaved).angles(pos)
+    cv = ops.Rotation(V, 5e3, interleaved).angles(pos)
+    res = []
+    for n in (T, 1000):
+        kc = torch.zeros(T // 16, 16, G, 256, dtype=dtype, device=dev)
+        vc = torch.zeros(T // 16, G, 128, 16, dtype=dtype, device=dev)
+        q = torch.cat([ops.rotary_qkv(
+            x[a:a + n], (0, H * D, (H + G) * D), H, G, D, V, pos[a:a + n], kc, vc, q_norm=w[0],
+            k_norm=w[1], cs_qk=ck[a:a + n], cs_v=cv[a:a + n], interleaved=interleaved)
+            for a in range(0, T, n)])
+        res.append((q, kc, vc))
+    for a, b in zip(*res):
+        assert torch.equal(a, b)
+    assert (res[0][1][..., :D] != 0).any(-1).all() and (res[0][2][:, :, :V] != 0).any(-1).all()
+
+
+@kinds
 @pytest.mark.parametrize("size,keep", [(17, 0), (64, 3), (48, 16), (128, 20), (5, 1)])
 @pytest.mark.parametrize("sizes", [[300], [1], [2, 31, 64]])
 def test_window_edges_show(dev, dtype, tol, size, keep, sizes):
